@@ -135,7 +135,96 @@ def dense_mlp(x, w, eps):
     return w["down"] @ poly_norm(w["up"] @ x, *w["act"], eps)
 
 
-MIXERS = {"mamba2": mamba2, "latent_attention": latent_attention}
+def layer_norm(x, w, eps):
+    d = x - np.mean(x)
+    return d / np.sqrt(np.mean(d * d) + eps) * w
+
+
+def distance_bucket(n, rows, top):
+    """the first half of the rows: one distance each; the second half: logarithmic steps up to `top`, the last row beyond"""
+    half = rows // 2
+    if n < half:
+        return n
+    return min(rows - 1, half + math.floor(math.log(n / half) / math.log(top / half) * (rows - half)))
+
+
+def visible(i, j, mask):
+    """position i sees position j: behind it, and within the window or among the first tokens that are kept"""
+    return j <= i and (i - j < mask["size"] or j < mask["keep_first"])
+
+
+def softcap(s, cap):
+    return cap * np.tanh(s / cap)
+
+
+def biased_softmax(s, bias):
+    e = np.exp(s + bias - np.max(s + bias))
+    return e / np.sum(e)
+
+
+def window_attention(h, st, mx, w, eps):
+    """one token through grouped-query attention over a window and the first tokens: unit-RMS queries and keys, capped scores, a bias per distance and head, a gate per
+    head; st = {k, v: every key and value so far}"""
+    H, G, d, dv = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+    q = (w["q"] @ h).reshape(H, d)
+    k = np.stack([rms(x, eps) for x in (w["k"] @ h).reshape(G, d)])
+    v = (w["v"] @ h).reshape(G, dv)
+    st["k"] = st.get("k", []) + [k]
+    st["v"] = st.get("v", []) + [v]
+    i = len(st["k"]) - 1
+    seen = [j for j in range(i + 1) if visible(i, j, mx["mask"])]
+    buckets = [distance_bucket(i - j, len(w["rel"]), mx["bias_max"]) for j in seen]
+    gate = sigmoid(w["g"] @ h)
+    K, V = np.stack([st["k"][j] for j in seen]), np.stack([st["v"][j] for j in seen])
+    o = np.zeros((H, dv))
+    for a in range(H):
+        g = a // (H // G)
+        s = softcap((K[:, g] @ rms(q[a], eps)) * mx["scale"], mx["softcap"])
+        o[a] = gate[a] * (biased_softmax(s, w["rel"][buckets, a]) @ V[:, g])
+    return w["o"] @ o.reshape(-1)
+
+
+def gla_decay(z, tau):
+    return sigmoid(z) ** (1.0 / tau)
+
+
+def gla_step(S, alpha, k, v, q):
+    """one token of one head: every row (key channel) of S [dim, vdim] decays by its own alpha, takes k v^T and is read by q"""
+    S = alpha[:, None] * S + np.outer(k, v)
+    return S, S.T @ q
+
+
+def gated_linear(h, st, mx, w, eps):
+    """one token through gated linear attention; st = {S}"""
+    H, d, dv = mx["heads"], mx["dim"], mx["vdim"]
+    if not st:
+        st["S"] = np.zeros((H, d, dv))
+    q, k, v = (w["q"] @ h).reshape(H, d) / math.sqrt(d), (w["k"] @ h).reshape(H, d), (w["v"] @ h).reshape(H, dv)
+    alpha = gla_decay(w["a2"] @ (w["a1"] @ h) + w["a2.b"], mx["tau"]).reshape(H, d)
+    o = np.zeros((H, dv))
+    for a in range(H):
+        st["S"][a], y = gla_step(st["S"][a], alpha[a], k[a], v[a], q[a])
+        o[a] = rms(y, eps) * w["norm"]
+    return w["o"] @ (o.reshape(-1) * silu(w["g"] @ h))
+
+
+def parallel(h, st, mx, w, eps):
+    """both mixers read the same input; their results are added with a scale each"""
+    part = lambda side: {k[len(side):]: v for k, v in w.items() if k.startswith(side)}
+    st.setdefault("left", {}); st.setdefault("right", {})
+    return mx["left_scale"] * window_attention(h, st["left"], mx["left"], part("left."), eps) + mx["right_scale"] * gated_linear(h, st["right"], mx["right"], part("right."), eps)
+
+
+def clamped_glu(gate, up, limit):
+    g, u = np.minimum(gate, limit), np.clip(up, -limit, limit)
+    return g * sigmoid(1.702 * g) * (u + 1)
+
+
+def glu_mlp(x, w, limit):
+    return w["down"] @ clamped_glu(w["gate"] @ x, w["up"] @ x, limit)
+
+
+MIXERS = {"mamba2": mamba2, "latent_attention": latent_attention, "parallel": parallel}
 
 
 # ---- model ---------------------------------------------------------------------------------------------------------------------------------
@@ -153,22 +242,37 @@ class StackModel:
     def load(cls, folder):
         return cls(json.load(open(folder + "/config.json")), read_safetensors(folder + "/model.safetensors"))
 
+    def tupitar_layer(self, x, ly, mix, mlp, top, st, eps):
+        """one number scales the norm of every sublayer's output; mixers read a blend of this token and the previous one"""
+        h = token_shift(x, st["prev"], top["shift"])
+        st["prev"] = x
+        x = x + scalar_norm(MIXERS[ly["type"]](h, st["mix"], ly["mixer"], mix, eps), top["norm1"], eps)
+        if ly["mlp"] is not None:
+            x = x + scalar_norm(dense_mlp(x, mlp, eps), top["norm2"], eps)
+        return x
+
+    def mafurax_layer(self, x, ly, mix, mlp, top, st, eps):
+        """a layer norm in front of every sublayer, another on its output, and a scale per element on that"""
+        x = x + layer_norm(MIXERS[ly["type"]](layer_norm(x, top["norm1"], eps), st["mix"], ly["mixer"], mix, eps), top["norm1b"], eps) * top["ls1"]
+        if ly["mlp"] is not None:
+            x = x + layer_norm(glu_mlp(layer_norm(x, top["norm2"], eps), mlp, ly["mlp"]["limit"]), top["norm2b"], eps) * top["ls2"]
+        return x
+
     def new_state(self):
         return {"n": 0, "layers": [{"prev": np.zeros(self.cfg["width"]), "mix": {}} for _ in self.layers]}
 
     def token(self, tok, state, trace=None):
         """one token; returns its logits and advances the state"""
         eps = self.cfg["norm"]["eps"]
-        x = self.w["embed"][tok] * self.cfg["embedding"]["scale"] + self.w["pos"][state["n"]]
+        mafurax = self.cfg["architecture"] == "Mafurax"
+        x = self.w["embed"][tok] if mafurax else self.w["embed"][tok] * self.cfg["embedding"]["scale"] + self.w["pos"][state["n"]]
         for (ly, mix, mlp, top), st in zip(self.layers, state["layers"]):
-            h = token_shift(x, st["prev"], top["shift"])
-            st["prev"] = x
-            x = x + scalar_norm(MIXERS[ly["type"]](h, st["mix"], ly["mixer"], mix, eps), top["norm1"], eps)
-            if ly["mlp"] is not None:
-                x = x + scalar_norm(dense_mlp(x, mlp, eps), top["norm2"], eps)
+            x = (self.mafurax_layer if mafurax else self.tupitar_layer)(x, ly, mix, mlp, top, st, eps)
             if trace is not None:
                 trace.append(x)
         state["n"] += 1
+        if mafurax:
+            return self.w["embed"] @ layer_norm(x, self.w["final.norm"], eps) * self.cfg["logit_scale"]
         return self.w["head"] @ scalar_norm(x, self.w["final.norm"], eps)
 
     def forward(self, tokens, state=None, trace=None):
@@ -178,13 +282,17 @@ class StackModel:
 
 
 # ---- small random models ---------------------------------------------------------------------------------------------------------------------
-def random_model(cfg, seed):
+def random_model(cfg, seed, rows=None):
     """bfloat16-representable weights of unit gain; decays, biases and gates spread so that no mechanism is idle"""
     r = np.random.default_rng(seed)
     E, V = cfg["width"], cfg["vocab"]
     lin = lambda o, i, s=1.0: r.standard_normal((o, i)) * s / math.sqrt(i)
-    w = {"embed": r.standard_normal((V, E)) / cfg["embedding"]["scale"], "pos": r.standard_normal((cfg["max_positions"], E)) * 0.3,
-         "final.norm": np.array(1.1), "head": lin(V, E)}
+    mafurax = cfg["architecture"] == "Mafurax"
+    if mafurax:
+        w = {"embed": lin(V, E, math.sqrt(E)), "final.norm": 1 + 0.2 * r.standard_normal(E)}
+    else:
+        w = {"embed": r.standard_normal((V, E)) / cfg["embedding"]["scale"], "pos": r.standard_normal((cfg["max_positions"], E)) * 0.3,
+             "final.norm": np.array(1.1), "head": lin(V, E)}
     for i, ly in enumerate(cfg["layers"]):
         p, mx = "l%d." % i, ly["mixer"]
         m = {}
@@ -193,11 +301,27 @@ def random_model(cfg, seed):
             ch = H * P + 2 * G * N
             m = {"in": lin(H * P + ch + H, E), "conv": r.standard_normal((ch, K)) / math.sqrt(K), "conv.b": r.standard_normal(ch) * 0.1,
                  "dt_bias": r.uniform(-4, 0, H), "A_log": r.uniform(-1, 1.5, H), "D": r.standard_normal(H), "norm": 1 + 0.2 * r.standard_normal(H * P), "o": lin(E, H * P)}
-        else:
+        elif ly["type"] == "latent_attention":
             H, d, dv, R = mx["heads"], mx["dim"], mx["vdim"], mx["kv_rank"]
             m = {"q": lin(H * d, E), "dkv": lin(R, E), "dkv.norm": 1 + 0.2 * r.standard_normal(R), "uk": lin(H * d, R, 2.0), "uv": lin(H * dv, R), "sink": r.standard_normal(H) + 1,
                  "g": lin(H, E), "o": lin(E, H * dv)}
+        else:
+            # sizes that the configuration does not name: bias rows, rank of the decays
+            a, b = mx["left"], mx["right"]
+            B, R = (rows or {}).get("rel", 8), (rows or {}).get("rank", 5)
+            H, G, d, dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            m = {"left.q": lin(H * d, E), "left.k": lin(G * d, E), "left.v": lin(G * dv, E), "left.rel": r.standard_normal((B, H)), "left.g": lin(H, E), "left.o": lin(E, H * dv)}
+            H, d, dv = b["heads"], b["dim"], b["vdim"]
+            m.update({"right.q": lin(H * d, E), "right.k": lin(H * d, E, 0.5), "right.v": lin(H * dv, E), "right.g": lin(H * dv, E), "right.o": lin(E, H * dv), "right.norm": 1 + 0.2 * r.standard_normal(dv),
+                      "right.a1": lin(R, E), "right.a2": lin(H * d, R, 2.0), "right.a2.b": r.uniform(-3, 6, H * d)})
         w.update({p + "mix." + k: v for k, v in m.items()})
+        if mafurax:
+            n = lambda: 1 + 0.2 * r.standard_normal(E)
+            w.update({p + "norm1": n(), p + "norm1b": n(), p + "ls1": r.uniform(0.3, 0.9, E) * r.choice([-1, 1], E)})
+            if ly["mlp"] is not None:
+                F = ly["mlp"]["ff"]
+                w.update({p + "norm2": n(), p + "norm2b": n(), p + "ls2": r.uniform(0.3, 0.9, E), p + "mlp.gate": lin(F, E), p + "mlp.up": lin(F, E), p + "mlp.down": lin(E, F)})
+            continue
         w[p + "norm1"] = np.array(r.uniform(0.4, 0.9)); w[p + "shift"] = r.uniform(0, 1, E)
         if ly["mlp"] is not None:
             F = ly["mlp"]["ff"]
