@@ -6,11 +6,23 @@
 #include <fstream>
 #include <iterator>
 
-static const bamd_stack_design TUPITAR = { true, true, STACK_NORM_OUTPUT_SCALAR, STACK_ACT_POLYNORM, "mamba2 latent_attention", true, true };
+static const bamd_stack_design TUPITAR = [] {
+    bamd_stack_design d = {};
+    d.scaled_embedding = d.learned_positions = d.token_shift = true; d.norm = STACK_NORM_OUTPUT_SCALAR; d.mlp_act = STACK_ACT_POLYNORM;
+    d.mixers = "mamba2 latent_attention"; d.latent_sink = d.latent_gate = true;
+    return d;
+}();
+static const bamd_stack_design MAFURAX = [] {
+    bamd_stack_design d = {};
+    d.norm = STACK_NORM_SANDWICH; d.mlp_act = STACK_ACT_CLAMPED_GLU; d.tied_head = true;
+    d.mixers = "parallel"; d.kv_unit = d.kv_cap = d.kv_bias = d.kv_gate = d.gla_gate = true;
+    return d;
+}();
 
 static const bamd_arch TABLE[] = {
     { "llama", false, bamd_llama_load, nullptr },
     { "Tupitar", true, bamd_stack_load, &TUPITAR },
+    { "Mafurax", true, bamd_stack_load, &MAFURAX },
 };
 
 const bamd_arch * bamd_arch_find(const std::string & name, bool folder) {

@@ -2,25 +2,26 @@
 //   dense_gemm_kernel: many rows (prompts).  Weight and activation tiles through two LDS stages in operand order (every LDS access is one contiguous kilobyte per
 //     wave), the next stage's global loads in flight under the matrix instructions.
 //   dense_mv_kernel: few rows (decoding).  The eight or sixteen waves of a block split K; every wave streams its share of a 16-row tile straight from HBM into matrix operands.  With
-//     a single row the mechanism in front of the product (residual + norm + token shift, PolyNorm, grouped norm, last norm) runs as its prologue, its weights
+//     a single row the mechanism in front of the product (residual + norm + token shift or layer norms, PolyNorm, clamped gated unit, grouped norm, last norm) runs as its prologue, its weights
 //     already requested.
 #include "bamd_dense_device.h"
 
-// ---- packing at load: value (row, col) of the packed matrix = src[row_off[row] + col_off[col]], zero where either is negative ---------------------------
-__global__ void __launch_bounds__(64) pack_kernel(const uint16_t * src, const int32_t * row_off, const int32_t * col_off, int k_tiles, uint16_t * dst) {
+// ---- packing at load: value (row, col) of the packed matrix = src[row_off[row] + col_off[col]], zero where either is negative; row tiles go to every step-th row tile of
+// a matrix of ld column blocks ------------------------------------------------------------------------------------------------------------------------------
+__global__ void __launch_bounds__(64) pack_kernel(const uint16_t * src, const int32_t * row_off, const int32_t * col_off, int k_tiles, uint16_t * dst, int step, int ld) {
     const int lane = threadIdx.x, kt = blockIdx.x % k_tiles, rt = blockIdx.x / k_tiles;
     const int ro = row_off[rt * 16 + (lane & 15)];
-    uint16_t * d = dst + ((size_t) blockIdx.x * 64 + lane) * 8;
+    uint16_t * d = dst + (((size_t) rt * step * ld + kt) * 64 + lane) * 8;
     for (int i = 0; i < 8; ++i) { const int co = col_off[kt * 32 + (lane >> 4) * 8 + i]; d[i] = ro < 0 || co < 0 ? 0 : src[(size_t) ro + co]; }
 }
-void bamd_launch_pack(const uint16_t * src, const int32_t * row_off, const int32_t * col_off, int row_tiles, int k_tiles, uint16_t * dst, hipStream_t s) {
-    hipLaunchKernelGGL(pack_kernel, dim3(row_tiles * k_tiles), dim3(64), 0, s, src, row_off, col_off, k_tiles, dst);
+void bamd_launch_pack(const uint16_t * src, const int32_t * row_off, const int32_t * col_off, int row_tiles, int k_tiles, uint16_t * dst, int step, int ld, hipStream_t s) {
+    hipLaunchKernelGGL(pack_kernel, dim3(row_tiles * k_tiles), dim3(64), 0, s, src, row_off, col_off, k_tiles, dst, step, ld);
 }
 
 // ---- many rows --------------------------------------------------------------------------------------------------------------------------------------
 // TM activation rows x TN matrix rows per block of four waves (2 x 2); KT 32-column blocks per stage
 template <typename T, int TM, int TN, int KT, int OUT>
-__global__ void __launch_bounds__(256) dense_gemm_kernel(bamd_dense w, const T * x, int ldx, int rows, void * out, int ldo, int n_mt, int n_nt) {
+__global__ void __launch_bounds__(256) dense_gemm_kernel(bamd_dense w, const T * x, int ldx, int rows, void * out, int ldo, int n_mt, int n_nt, float limit) {
     constexpr int FB = 64 * 8 * sizeof(T);                        // bytes of one operand block (16 rows x 32 columns)
     constexpr int XT = TM / 16, WT = TN / 16, XC = XT * KT * FB / 4096, WC = WT * KT * 1024 / 4096;   // 16-byte pieces per thread and stage
     constexpr int WF = 1024;                                      // weights stay bfloat16 in LDS
@@ -103,6 +104,13 @@ __global__ void __launch_bounds__(256) dense_gemm_kernel(bamd_dense w, const T *
                 if (n >= w.rows) continue;
 #pragma unroll
                 for (int k = 0; k < 4; ++k) if (m + k < rows) ((T *) out)[(size_t) n * ldo + m + k] = to_act<T>(acc[i][j][k]);
+            } else if constexpr (OUT == BAMD_OUT_GLU) {           // tiles in turn: gate, up
+                const int n = (nb >> 1) + (lane >> 4) * 4, m = mb + (lane & 15);
+                if ((j & 1) || m >= rows) continue;
+                bamd_v4 o;
+#pragma unroll
+                for (int k = 0; k < 4; ++k) o[k] = clamped_glu(acc[i][j][k], acc[i][j | 1][k], limit);
+                store4<T>((T *) out + (size_t) m * ldo + n, o);
             } else {
                 const int n = nb + (lane >> 4) * 4, m = mb + (lane & 15);
                 if (m >= rows) continue;
@@ -119,22 +127,31 @@ __global__ void __launch_bounds__(256) dense_gemm_kernel(bamd_dense w, const T *
         }
 }
 template <typename T, int TM, int TN, int KT, int OUT>
-static int gemm_go(const bamd_dense & w, const void * x, int ldx, int rows, void * out, int ldo, hipStream_t s) {
+static int gemm_go(const bamd_dense & w, const void * x, int ldx, int rows, void * out, int ldo, float limit, hipStream_t s) {
     const int n_mt = (rows + TM - 1) / TM, n_nt = (w.row_tiles + TN / 16 - 1) / (TN / 16), per = (n_mt * n_nt + 7) / 8;
     const size_t lds = 2 * ((size_t) TM / 16 * KT * 64 * 8 * sizeof(T) + (size_t) TN / 16 * KT * 1024);
-    hipLaunchKernelGGL((dense_gemm_kernel<T, TM, TN, KT, OUT>), dim3(per * 8), dim3(256), lds, s, w, (const T *) x, ldx, rows, out, ldo, n_mt, n_nt);
+    hipLaunchKernelGGL((dense_gemm_kernel<T, TM, TN, KT, OUT>), dim3(per * 8), dim3(256), lds, s, w, (const T *) x, ldx, rows, out, ldo, n_mt, n_nt, limit);
     return 0;
 }
 template <typename T, int OUT>
-static int gemm_tiles(const bamd_dense & w, const void * x, int ldx, int rows, void * out, int ldo, hipStream_t s) {
-    if constexpr (sizeof(T) == 2) if ((long) ((rows + 127) / 128) * ((w.row_tiles + 7) / 8) >= 192) return gemm_go<T, 128, 128, 2, OUT>(w, x, ldx, rows, out, ldo, s);
-    return gemm_go<T, 64, 64, sizeof(T) == 2 ? 4 : 2, OUT>(w, x, ldx, rows, out, ldo, s);
+static int gemm_tiles(const bamd_dense & w, const void * x, int ldx, int rows, void * out, int ldo, float limit, hipStream_t s) {
+    if constexpr (sizeof(T) == 2) if ((long) ((rows + 127) / 128) * ((w.row_tiles + 7) / 8) >= 192) return gemm_go<T, 128, 128, 2, OUT>(w, x, ldx, rows, out, ldo, limit, s);
+    return gemm_go<T, 64, 64, sizeof(T) == 2 ? 4 : 2, OUT>(w, x, ldx, rows, out, ldo, limit, s);
 }
 // f32 rows are stored four matrix rows at a time: ldo % 4 == 0; x rows start on 16 bytes and hold k_tiles * 32 columns
-int bamd_launch_dense_gemm(int act, const bamd_dense & w, const void * x, int ldx, int rows, void * out, int ldo, int kind, hipStream_t s) {
+template <typename T>
+static int gemm_out(const bamd_dense & w, const void * x, int ldx, int rows, void * out, int ldo, int kind, float limit, hipStream_t s) {
+    switch (kind) {
+        case BAMD_OUT_F32: return gemm_tiles<T, BAMD_OUT_F32>(w, x, ldx, rows, out, ldo, limit, s);
+        case BAMD_OUT_ACT: return gemm_tiles<T, BAMD_OUT_ACT>(w, x, ldx, rows, out, ldo, limit, s);
+        case BAMD_OUT_ACT_T: return gemm_tiles<T, BAMD_OUT_ACT_T>(w, x, ldx, rows, out, ldo, limit, s);
+        case BAMD_OUT_GLU: return (w.row_tiles & 1) || ldo < w.row_tiles * 8 ? 1 : gemm_tiles<T, BAMD_OUT_GLU>(w, x, ldx, rows, out, ldo, limit, s);
+    }
+    return 1;
+}
+int bamd_launch_dense_gemm(int act, const bamd_dense & w, const void * x, int ldx, int rows, void * out, int ldo, int kind, hipStream_t s, float limit) {
     if (rows < 1 || w.row_tiles < 1 || w.k_tiles < 1 || ldx < w.k_tiles * 32 || (ldx & 7) || (ldo & 3)) return 1;
-    if (act == BAMD_ACT_F32) return kind == BAMD_OUT_F32 ? gemm_tiles<float, BAMD_OUT_F32>(w, x, ldx, rows, out, ldo, s) : kind == BAMD_OUT_ACT ? gemm_tiles<float, BAMD_OUT_ACT>(w, x, ldx, rows, out, ldo, s) : gemm_tiles<float, BAMD_OUT_ACT_T>(w, x, ldx, rows, out, ldo, s);
-    return kind == BAMD_OUT_F32 ? gemm_tiles<bamd_bf, BAMD_OUT_F32>(w, x, ldx, rows, out, ldo, s) : kind == BAMD_OUT_ACT ? gemm_tiles<bamd_bf, BAMD_OUT_ACT>(w, x, ldx, rows, out, ldo, s) : gemm_tiles<bamd_bf, BAMD_OUT_ACT_T>(w, x, ldx, rows, out, ldo, s);
+    return act == BAMD_ACT_F32 ? gemm_out<float>(w, x, ldx, rows, out, ldo, kind, limit, s) : gemm_out<bamd_bf>(w, x, ldx, rows, out, ldo, kind, limit, s);
 }
 
 // ---- few rows ---------------------------------------------------------------------------------------------------------------------------------------
@@ -159,6 +176,8 @@ __global__ void __launch_bounds__(64 * NW) dense_mv_kernel(bamd_dense w, bamd_ba
         if constexpr (PRE == BAMD_PRE_RESIDUAL) residual_row<T, true>(b, p.res, 0, h, blockIdx.x == 0, red);
         if constexpr (PRE == BAMD_PRE_POLY) poly_row<T>(p.poly, 0, h, red);
         if constexpr (PRE == BAMD_PRE_GROUP) group_norm_row<T>(p.grp, 0, h, red);
+        if constexpr (PRE == BAMD_PRE_GLU) glu_row<T>(p.glu, 0, h);
+        if constexpr (PRE == BAMD_PRE_LAYER) layer_row<T>(p.res, p.want ? p.want[0] : 0, p.want ? p.gf : p.res.gi, h, !p.want && blockIdx.x == 0, red);
         if constexpr (PRE == BAMD_PRE_FINAL) final_row<T>(p.res, p.want[0], p.gf, h, red);
         __syncthreads();
     }
@@ -220,11 +239,13 @@ template <typename T>
 static int mv_pick(const bamd_dense & w, int pre, const bamd_batch_dev & b, const bamd_pre_args & p, const void * x, int ldx, int rows, float * out, int ldo, hipStream_t s) {
     if (pre != BAMD_PRE_ROWS) {
         if (rows != 1 || bamd_dense_mv_lds(sizeof(T) == 4 ? BAMD_ACT_F32 : BAMD_ACT_BF16, w.k_tiles * 32) > BAMD_MV_LDS) return 1;
-        const int ldh = pre == BAMD_PRE_POLY ? p.poly.ldh : pre == BAMD_PRE_GROUP ? p.grp.ldh : p.res.ldh;
+        const int ldh = pre == BAMD_PRE_POLY ? p.poly.ldh : pre == BAMD_PRE_GROUP ? p.grp.ldh : pre == BAMD_PRE_GLU ? p.glu.ldh : p.res.ldh;
         if (ldh != w.k_tiles * 32) return 1;
-        if (pre == BAMD_PRE_RESIDUAL) mv_one<T, BAMD_PRE_RESIDUAL>(w, b, p, x, ldx, rows, out, ldo, s);
+        if (pre == BAMD_PRE_RESIDUAL && p.res.norm != BAMD_NORM_LAYER) mv_one<T, BAMD_PRE_RESIDUAL>(w, b, p, x, ldx, rows, out, ldo, s);
         else if (pre == BAMD_PRE_POLY) mv_one<T, BAMD_PRE_POLY>(w, b, p, x, ldx, rows, out, ldo, s);
         else if (pre == BAMD_PRE_GROUP) mv_one<T, BAMD_PRE_GROUP>(w, b, p, x, ldx, rows, out, ldo, s);
+        else if (pre == BAMD_PRE_GLU) mv_one<T, BAMD_PRE_GLU>(w, b, p, x, ldx, rows, out, ldo, s);
+        else if (p.res.norm == BAMD_NORM_LAYER) mv_one<T, BAMD_PRE_LAYER>(w, b, p, x, ldx, rows, out, ldo, s);
         else mv_one<T, BAMD_PRE_FINAL>(w, b, p, x, ldx, rows, out, ldo, s);
         return 0;
     }

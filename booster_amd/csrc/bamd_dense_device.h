@@ -20,6 +20,7 @@ template <> struct Frag<bamd_bf> {
     __device__ __forceinline__ void load(const bamd_bf * p) { v = *(const bamd_bf8 *) p; }
     __device__ __forceinline__ void weight(bamd_u4 w) { v = __builtin_bit_cast(bamd_bf8, w); }
     __device__ __forceinline__ void set(int i, float f) { v[i] = (bamd_bf) f; }
+    __device__ __forceinline__ void store(bamd_bf * p) const { *(bamd_bf8 *) p = v; }
 };
 template <> struct Frag<float> {
     bamd_v4 a, b;
@@ -27,6 +28,7 @@ template <> struct Frag<float> {
     __device__ __forceinline__ void load(const float * p) { a = *(const bamd_v4 *) p; b = *(const bamd_v4 *) (p + 4); }
     __device__ __forceinline__ void weight(bamd_u4 w) { a = bamd_v4{ bf_lo(w.x), bf_hi(w.x), bf_lo(w.y), bf_hi(w.y) }; b = bamd_v4{ bf_lo(w.z), bf_hi(w.z), bf_lo(w.w), bf_hi(w.w) }; }
     __device__ __forceinline__ void set(int i, float f) { if (i < 4) a[i] = f; else b[i - 4] = f; }
+    __device__ __forceinline__ void store(float * p) const { *(bamd_v4 *) p = a; *(bamd_v4 *) (p + 4) = b; }
 };
 // D[row = (lane / 16) * 4 + i][col = lane % 16] += sum over 32 k of A[row][k] B[k][col]
 __device__ __forceinline__ bamd_v4 mma(const Frag<bamd_bf> & a, const Frag<bamd_bf> & b, bamd_v4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0); }
@@ -43,13 +45,37 @@ __device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf
 __device__ __forceinline__ float silu_f(float x) { return x / (1.0f + expf(-x)); }
 __device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x))); }
 
+// sum over the wave, the same in every lane: rows of sixteen lanes by data-parallel moves, then the four rows
+__device__ __forceinline__ float wave_sum(float v) {
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xb1, 0xf, 0xf, true));      // lane ^ 1
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4e, 0xf, 0xf, true));      // lane ^ 2
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xf, 0xf, true));     // the other four of eight
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140, 0xf, 0xf, true));     // the other eight of sixteen
+    const int i = __float_as_int(v);
+    return (__int_as_float(__builtin_amdgcn_readlane(i, 0)) + __int_as_float(__builtin_amdgcn_readlane(i, 16))) + (__int_as_float(__builtin_amdgcn_readlane(i, 32)) + __int_as_float(__builtin_amdgcn_readlane(i, 48)));
+}
+// maximum and sum over the sixteen lanes of a row
+__device__ __forceinline__ float row_sum16(float v) {
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xb1, 0xf, 0xf, true));
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4e, 0xf, 0xf, true));
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xf, 0xf, true));
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140, 0xf, 0xf, true));
+    return v;
+}
+__device__ __forceinline__ float row_max16(float v) {
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xb1, 0xf, 0xf, true)));
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4e, 0xf, 0xf, true)));
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xf, 0xf, true)));
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140, 0xf, 0xf, true)));
+    return v;
+}
+__device__ __forceinline__ void wave_lds_fence() { __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront"); __builtin_amdgcn_wave_barrier(); }
+
 // sums of NV values over the block; red: NV * 16 floats of LDS.  Every thread gets the result
 template <int NV> __device__ __forceinline__ void block_sum(float (&v)[NV], float * red) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = (blockDim.x + 63) >> 6;
 #pragma unroll
-    for (int i = 0; i < NV; ++i)
-#pragma unroll
-        for (int o = 32; o > 0; o >>= 1) v[i] += __shfl_xor(v[i], o);
+    for (int i = 0; i < NV; ++i) v[i] = wave_sum(v[i]);
     __syncthreads();
     if (lane == 0)
 #pragma unroll
@@ -89,6 +115,106 @@ template <> __device__ __forceinline__ void store4<bamd_bf>(bamd_bf * h, bamd_v4
     *(bf4 *) h = bf4{ (bamd_bf) v[0], (bamd_bf) v[1], (bamd_bf) v[2], (bamd_bf) v[3] };
 }
 template <typename T> __device__ __forceinline__ void zero_tail(T * h, int n, int ld) { for (int i = n + threadIdx.x; i < ld; i += blockDim.x) h[i] = to_act<T>(0.f); }
+
+// mean and variance (mean of the squared deviations) of a row in registers: per wave around its own mean, then over the waves.  red: 48 floats of LDS
+template <int RC> __device__ __forceinline__ void row_moments(const RowRegs<RC> & r, int n, float * red, float & mean, float & var) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    float s = 0.f, c = 0.f, q = 0.f;
+#pragma unroll
+    for (int i = 0; i < RC; ++i) if (RowRegs<RC>::at(i) < n) { s += (r.v[i][0] + r.v[i][1]) + (r.v[i][2] + r.v[i][3]); c += 4.f; }
+    s = wave_sum(s); c = wave_sum(c);
+    const float m = c > 0.f ? s / c : 0.f;
+#pragma unroll
+    for (int i = 0; i < RC; ++i) if (RowRegs<RC>::at(i) < n)
+#pragma unroll
+        for (int k = 0; k < 4; ++k) { const float d = r.v[i][k] - m; q += d * d; }
+    q = wave_sum(q);
+    __syncthreads();
+    if (lane == 0) { red[wave] = m; red[16 + wave] = q; red[32 + wave] = c; }
+    __syncthreads();
+    mean = 0.f; var = 0.f;
+    for (int w = 0; w < nw; ++w) mean += red[w] * red[32 + w];
+    mean /= (float) n;
+    for (int w = 0; w < nw; ++w) { const float d = red[w] - mean; var += red[16 + w] + red[32 + w] * d * d; }
+    var /= (float) n;
+}
+// residual sum with the layer norm of the sublayer's output, and the layer norm (gain gi, null: none) the next sublayer reads, of one row by the whole block
+template <typename T>
+__device__ __forceinline__ void layer_row(const bamd_residual_args & a, int row, const float * gi, T * h, bool write, float * red) {
+    constexpr int RC = 2;
+    const int E = a.E;
+    const float * x = a.x + (size_t) row * E, * y = a.y ? a.y + (size_t) row * a.ldy : nullptr;
+    float * xo = a.xo + (size_t) row * E;
+    if (RowRegs<RC>::fits(E)) {
+        RowRegs<RC> xr, yr;
+        bamd_v4 g[RC], w[RC];
+        xr.load(x, E);
+        if (y) yr.load(y, E);
+#pragma unroll
+        for (int c = 0; c < RC; ++c) {
+            const int i = RowRegs<RC>::at(c);
+            if (y) g[c] = i < E ? *(const bamd_v4 *) (a.g + i) : bamd_v4{ 0, 0, 0, 0 };
+            if (gi) w[c] = i < E ? *(const bamd_v4 *) (gi + i) : bamd_v4{ 0, 0, 0, 0 };
+        }
+        float mean, var;
+        if (y) {
+            row_moments<RC>(yr, E, red, mean, var);
+            const float r = 1.0f / sqrtf(var + a.eps);
+#pragma unroll
+            for (int c = 0; c < RC; ++c) xr.v[c] = xr.v[c] + (yr.v[c] - mean) * r * g[c];
+        }
+        if (write)
+#pragma unroll
+            for (int c = 0; c < RC; ++c) { const int i = RowRegs<RC>::at(c); if (i < E) *(bamd_v4 *) (xo + i) = xr.v[c]; }
+        if (!h) return;
+        float r = 1.f;
+        mean = 0.f;
+        if (gi) { row_moments<RC>(xr, E, red, mean, var); r = 1.0f / sqrtf(var + a.eps); }
+#pragma unroll
+        for (int c = 0; c < RC; ++c) { const int i = RowRegs<RC>::at(c); if (i < E) store4<T>(h + i, gi ? (xr.v[c] - mean) * r * w[c] : xr.v[c]); }
+        zero_tail(h, E, a.ldh);
+        return;
+    }
+    float my = 0.f, ry = 0.f, v[1];
+    if (y) {
+        v[0] = 0.f;
+        for (int i = threadIdx.x; i < E; i += blockDim.x) v[0] += y[i];
+        block_sum<1>(v, red);
+        my = v[0] / (float) E; v[0] = 0.f;
+        for (int i = threadIdx.x; i < E; i += blockDim.x) { const float d = y[i] - my; v[0] += d * d; }
+        block_sum<1>(v, red);
+        ry = 1.0f / sqrtf(v[0] / (float) E + a.eps);
+    }
+    auto at = [&](int i) { return y ? x[i] + (y[i] - my) * ry * a.g[i] : x[i]; };
+    float mx = 0.f, rx = 1.f;
+    if (gi && h) {
+        v[0] = 0.f;
+        for (int i = threadIdx.x; i < E; i += blockDim.x) v[0] += at(i);
+        block_sum<1>(v, red);
+        mx = v[0] / (float) E; v[0] = 0.f;
+        for (int i = threadIdx.x; i < E; i += blockDim.x) { const float d = at(i) - mx; v[0] += d * d; }
+        block_sum<1>(v, red);
+        rx = 1.0f / sqrtf(v[0] / (float) E + a.eps);
+    }
+    for (int i = threadIdx.x; i < E; i += blockDim.x) {
+        const float xn = at(i);
+        if (write) xo[i] = xn;
+        if (h) h[i] = to_act<T>(gi ? (xn - mx) * rx * gi[i] : xn);
+    }
+    if (h) zero_tail(h, E, a.ldh);
+}
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
+}
+template <typename T>
+__device__ __forceinline__ void glu_row(const bamd_glu_args & a, int row, T * h) {
+    const float * z = a.z + (size_t) row * a.ldz;
+    for (int i = threadIdx.x * 4; i < a.ldh; i += blockDim.x * 4) {
+        const bamd_v4 g = *(const bamd_v4 *) (z + (i >> 4) * 32 + (i & 15)), u = *(const bamd_v4 *) (z + (i >> 4) * 32 + 16 + (i & 15));
+        store4<T>(h + i, bamd_v4{ clamped_glu(g[0], u[0], a.limit), clamped_glu(g[1], u[1], a.limit), clamped_glu(g[2], u[2], a.limit), clamped_glu(g[3], u[3], a.limit) });
+    }
+}
 
 // residual sum, norm of the sublayer's output and token shift of one row by the whole block.  h: LDS or global row (null: none).  write: this block also stores x' and the
 // state.  SINGLE: the step has one row

@@ -7,8 +7,6 @@
 #include "bamd_dense_device.h"
 #include <math.h>
 
-__device__ __forceinline__ void wave_lds_fence() { __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront"); __builtin_amdgcn_wave_barrier(); }
-
 // ---- the cache --------------------------------------------------------------------------------------------------------------------------------------
 template <typename T> __device__ __forceinline__ void latent_store_row(const bamd_batch_dev & b, const bamd_latent_args & a, int row, float * red) {
     const bamd_entry e = b.ent[b.row_entry[row]];

@@ -1,5 +1,5 @@
 // bamd_rows.hip — row-wise mechanisms of the configured layer stacks, one block per row: embedding with learned positions, residual sum with the norm of the
-// sublayer's output and token shift, PolyNorm, grouped norm, the model's last norm, arg-max, and the device side of the greedy loop.  With a single row the same
+// sublayer's output and token shift (or layer norms in front and behind), PolyNorm, clamped gated unit, grouped norm, the model's last norm, arg-max, and the device side of the greedy loop.  With a single row the same
 // device functions run as the prologue of the product behind them (bamd_dense.hip).
 #include "bamd_dense_device.h"
 
@@ -23,6 +23,12 @@ template <typename T> __global__ void __launch_bounds__(1024) final_rows_kernel(
     __shared__ float red[64];
     final_row<T>(a, want[blockIdx.x], gf, (T *) a.h + (size_t) blockIdx.x * a.ldh, red);
 }
+template <typename T> __global__ void __launch_bounds__(1024) layer_rows_kernel(bamd_residual_args a, const int32_t * want, const float * gi) {
+    __shared__ float red[64];
+    const int row = want ? want[blockIdx.x] : blockIdx.x;
+    layer_row<T>(a, row, gi, a.h ? (T *) a.h + (size_t) blockIdx.x * a.ldh : nullptr, !want, red);
+}
+template <typename T> __global__ void __launch_bounds__(256) glu_rows_kernel(bamd_glu_args a) { glu_row<T>(a, blockIdx.x, (T *) a.h + (size_t) blockIdx.x * a.ldh); }
 template <typename T> __global__ void __launch_bounds__(1024) poly_rows_kernel(bamd_poly_args a) {
     __shared__ float red[64];
     poly_row<T>(a, blockIdx.x, (T *) a.h + (size_t) blockIdx.x * a.ldh, red);
@@ -68,16 +74,26 @@ void bamd_launch_embed_rows(const bamd_batch_dev & b, const uint16_t * embd, con
     hipLaunchKernelGGL(embed_rows_kernel, dim3((E + 1023) / 1024, b.rows), dim3(256), 0, s, b, embd, pos, scale, E, V, x);
 }
 void bamd_launch_residual_rows(int act, const bamd_batch_dev & b, const bamd_residual_args & a, hipStream_t s) {
-    if (act == BAMD_ACT_F32) hipLaunchKernelGGL(residual_rows_kernel<float>, dim3(b.rows), row_block(a.E), 0, s, b, a);
+    if (a.norm == BAMD_NORM_LAYER) {
+        if (act == BAMD_ACT_F32) hipLaunchKernelGGL(layer_rows_kernel<float>, dim3(b.rows), row_block(a.E), 0, s, a, nullptr, a.gi);
+        else hipLaunchKernelGGL(layer_rows_kernel<bamd_bf>, dim3(b.rows), row_block(a.E), 0, s, a, nullptr, a.gi);
+    } else if (act == BAMD_ACT_F32) hipLaunchKernelGGL(residual_rows_kernel<float>, dim3(b.rows), row_block(a.E), 0, s, b, a);
     else hipLaunchKernelGGL(residual_rows_kernel<bamd_bf>, dim3(b.rows), row_block(a.E), 0, s, b, a);
 }
 void bamd_launch_final_rows(int act, const bamd_residual_args & a, const int32_t * want, int n_want, const float * gf, hipStream_t s) {
-    if (act == BAMD_ACT_F32) hipLaunchKernelGGL(final_rows_kernel<float>, dim3(n_want), row_block(a.E), 0, s, a, want, gf);
+    if (a.norm == BAMD_NORM_LAYER) {
+        if (act == BAMD_ACT_F32) hipLaunchKernelGGL(layer_rows_kernel<float>, dim3(n_want), row_block(a.E), 0, s, a, want, gf);
+        else hipLaunchKernelGGL(layer_rows_kernel<bamd_bf>, dim3(n_want), row_block(a.E), 0, s, a, want, gf);
+    } else if (act == BAMD_ACT_F32) hipLaunchKernelGGL(final_rows_kernel<float>, dim3(n_want), row_block(a.E), 0, s, a, want, gf);
     else hipLaunchKernelGGL(final_rows_kernel<bamd_bf>, dim3(n_want), row_block(a.E), 0, s, a, want, gf);
 }
 void bamd_launch_poly_rows(int act, int rows, const bamd_poly_args & a, hipStream_t s) {
     if (act == BAMD_ACT_F32) hipLaunchKernelGGL(poly_rows_kernel<float>, dim3(rows), row_block(a.F), 0, s, a);
     else hipLaunchKernelGGL(poly_rows_kernel<bamd_bf>, dim3(rows), row_block(a.F), 0, s, a);
+}
+void bamd_launch_glu_rows(int act, int rows, const bamd_glu_args & a, hipStream_t s) {
+    if (act == BAMD_ACT_F32) hipLaunchKernelGGL(glu_rows_kernel<float>, dim3(rows), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(glu_rows_kernel<bamd_bf>, dim3(rows), dim3(256), 0, s, a);
 }
 void bamd_launch_group_norm_rows(int act, int rows, const bamd_group_norm_args & a, hipStream_t s) {
     if (act == BAMD_ACT_F32) hipLaunchKernelGGL(group_norm_rows_kernel<float>, dim3(rows), row_block(a.n), 0, s, a);

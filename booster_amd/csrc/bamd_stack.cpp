@@ -18,7 +18,7 @@
 #include <math.h>
 #include <string.h>
 
-void bamd_launch_pack(const uint16_t * src, const int32_t * row_off, const int32_t * col_off, int row_tiles, int k_tiles, uint16_t * dst, hipStream_t s);
+void bamd_launch_pack(const uint16_t * src, const int32_t * row_off, const int32_t * col_off, int row_tiles, int k_tiles, uint16_t * dst, int step, int ld, hipStream_t s);
 
 namespace {
 // BAMD_STAGE_GRAPH=0: decoding rows are enqueued kernel by kernel instead of as a captured hipGraph (as bamd_stage_step of the GGUF pipeline)
@@ -40,19 +40,31 @@ struct Loader {
         if (t->dtype != "BF16" && t->dtype != "F32") { fail("tensor " + name + ": type " + t->dtype + " not supported (BF16, F32)"); return nullptr; }
         return t;
     }
-    // 32-bit vector on the device
-    int vec(const std::string & name, std::vector<int64_t> shape, float ** out) {
+    // 32-bit values of a tensor
+    int values(const std::string & name, std::vector<int64_t> shape, std::vector<float> & h) {
         const SafeTensor * t = get(name, shape);
         if (!t) return 1;
-        std::vector<float> h((size_t) t->count());
+        h.resize((size_t) t->count());
         for (size_t i = 0; i < h.size(); ++i) {
             if (t->dtype == "F32") memcpy(&h[i], t->data + 4 * i, 4);
             else { uint16_t u; memcpy(&u, t->data + 2 * i, 2); const uint32_t w = (uint32_t) u << 16; memcpy(&h[i], &w, 4); }
         }
-        if (dev_alloc(m->allocs, (void **) out, std::max<size_t>(h.size(), 1) * 4)) return 1;
-        HIPC(hipMemcpy(*out, h.data(), h.size() * 4, hipMemcpyHostToDevice));
         return 0;
     }
+    template <typename U> int upload(const std::vector<U> & h, U ** out) {
+        if (dev_alloc(m->allocs, (void **) out, std::max<size_t>(h.size(), 1) * sizeof(U))) return 1;
+        HIPC(hipMemcpy(*out, h.data(), h.size() * sizeof(U), hipMemcpyHostToDevice));
+        return 0;
+    }
+    // 32-bit vector on the device, times a constant; by: times another tensor of the same shape
+    int vec(const std::string & name, std::vector<int64_t> shape, float ** out, float scale = 1.f, const std::string & by = "") {
+        std::vector<float> h, w;
+        if (values(name, shape, h) || (!by.empty() && values(by, shape, w))) return 1;
+        for (size_t i = 0; i < h.size(); ++i) h[i] *= w.empty() ? scale : w[i] * scale;
+        return upload(h, out);
+    }
+    // size of a tensor's dimension that no configuration entry names (0: no such tensor)
+    int dim(const std::string & name, size_t at) { const SafeTensor * t = file.find(name); return t && at < t->shape.size() && t->shape[at] > 0 && t->shape[at] < (1 << 28) ? (int) t->shape[at] : 0; }
     int raw(const std::string & name, std::vector<int64_t> shape, uint16_t ** out) {
         const SafeTensor * t = matrix(name, shape);
         if (!t) return 1;
@@ -66,8 +78,8 @@ struct Loader {
         if (t && t->count() > 0x7fffffffll) { fail("tensor " + name + ": more than 2^31 values"); return nullptr; }
         return t;
     }
-    // rows / columns of the packed matrix taken from the tensor's values at row[i] + col[j] (-1: zero), at tile row `tile0` of d
-    int pack(const SafeTensor * t, const std::vector<int32_t> & row, const std::vector<int32_t> & col, uint16_t * dst) {
+    // rows / columns of the packed matrix taken from the tensor's values at row[i] + col[j] (-1: zero); step: row tiles go to every step-th one, ld: column blocks of the whole matrix
+    int pack(const SafeTensor * t, const std::vector<int32_t> & row, const std::vector<int32_t> & col, uint16_t * dst, int step = 1, int ld = 0) {
         const int rt = up((int) row.size(), 16) / 16, kt = up((int) col.size(), 32) / 32;
         if (t->nbytes > staging_bytes) {
             if (staging) HIPC(hipFree(staging));
@@ -80,7 +92,7 @@ struct Loader {
         std::copy(col.begin(), col.end(), h.begin() + (size_t) rt * 16);
         HIPC(hipMemcpyAsync(staging, t->data, t->nbytes, hipMemcpyHostToDevice, s));
         HIPC(hipMemcpyAsync(maps, h.data(), n * 4, hipMemcpyHostToDevice, s));
-        bamd_launch_pack((const uint16_t *) staging, maps, maps + (size_t) rt * 16, rt, kt, dst, s);
+        bamd_launch_pack((const uint16_t *) staging, maps, maps + (size_t) rt * 16, rt, kt, dst, step, ld ? ld : kt, s);
         HIPC(hipGetLastError());
         HIPC(hipStreamSynchronize(s));
         m->weight_bytes += (int64_t) t->nbytes;
@@ -122,7 +134,7 @@ struct Conf {                                      // required entries of a JSON
 
 // ---- model --------------------------------------------------------------------------------------------------------------------------------------------
 struct Ctx; struct Pass;
-struct MixState { float * a = nullptr, * b = nullptr; void * cache = nullptr; };       // of one layer in one context
+struct MixState { float * a = nullptr, * b = nullptr; void * cache = nullptr, * cache2 = nullptr; std::vector<MixState> sub; };       // of one layer in one context
 struct Operand { int pre = BAMD_PRE_ROWS; bamd_group_norm_args grp; const void * x = nullptr; int ldx = 0; };   // what the output projection reads
 
 struct Mixer {
@@ -133,9 +145,12 @@ struct Mixer {
     virtual int run(Pass & p, MixState & st, Operand & o) = 0;       // p.y holds the input projection's rows
     virtual int f32_cols() const { return 0; }                       // columns of the f32 scratch row it wants
     virtual int latents() const { return 0; }
+    virtual int prompt_rows(int) const { return 0; }                 // query rows per tile of a prompt (0: no attention)
+    virtual int scan_blocks() const { return 0; }                    // blocks of one segment of a prompt's scan (0: no segments)
+    virtual void partials(int, size_t &, size_t &) const {}          // floats of the decoding shares' sums and of their maxima, for so many rows
     virtual double step_bytes(int len) const = 0;                    // state bytes of one decoded token
 };
-struct Layer { std::unique_ptr<Mixer> mix; float * norm1 = nullptr, * norm2 = nullptr, * shift = nullptr, * act = nullptr; bool mlp = false; bamd_dense up, down; int F = 0; };
+struct Layer { std::unique_ptr<Mixer> mix; float * norm1 = nullptr, * norm2 = nullptr, * pre1 = nullptr, * pre2 = nullptr, * shift = nullptr, * act = nullptr; bool mlp = false; bamd_dense up, down; int F = 0; float limit = 0; };      // norm: of a sublayer's output (scale included), pre: of its input
 
 struct Stack : bamd_arch_runtime {
     bamd_stack_design d; bamd_model * m = nullptr;
@@ -164,6 +179,8 @@ struct Timer {                                     // per-launch HIP events (pro
     ~Timer() { for (auto e : ev) hipEventDestroy(e); }
 };
 #define STACK_ROWS 2048                            /* token rows of one pass */
+#define SEG_MIN 64                                 /* tokens of the shortest scan segment */
+#define SEG_BLOCKS 768                             /* blocks a scan wants */
 struct Ctx {
     bamd_context * c = nullptr; Stack * st = nullptr;
     std::vector<Seq> seqs; std::vector<int32_t> free_pages; int max_pages = 0; bool pages_dirty = true;
@@ -174,9 +191,10 @@ struct Ctx {
     void * qp = nullptr; float * part_o = nullptr, * part_ml = nullptr;
     void * kc = nullptr, * kk = nullptr, * kv = nullptr; size_t kc_n = 0, kk_n = 0, kv_n = 0;      // unpacked latents / keys / values of a prompt pass
     float * filtered = nullptr, * steps = nullptr; size_t filtered_n = 0, steps_n = 0;             // filtered channels, step sizes and decays of a prompt pass
+    float * alpha = nullptr, * seg_state = nullptr, * seg_decay = nullptr; size_t alpha_n = 0, seg_state_n = 0, seg_decay_n = 0;      // decays and segment states of a prompt pass
     unsigned long long * keys = nullptr; int32_t * step = nullptr, * gen_out = nullptr; int gen_cap = 0;
-    // step descriptors: entries | row_entry | tokens | want | query tiles | key blocks, one device block per pass, filled from a ring of pinned blocks
-    struct Layout { size_t ent, row, tok, want, tile, kblk, total; int tiles, kblks; } lay;
+    // step descriptors: entries | row_entry | tokens | want | query tiles | key blocks | scan segments, one device block per pass, filled from a ring of pinned blocks
+    struct Layout { size_t ent, row, tok, want, tile, kblk, seg, total; int tiles, kblks, segs; } lay;
     unsigned char * dev = nullptr; int32_t * pages = nullptr;
     static constexpr int RING = 4;
     unsigned char * host[RING] = {}; int32_t * pages_host[RING] = {}; hipEvent_t ev[RING] = {}; int ring = 0;
@@ -184,13 +202,14 @@ struct Ctx {
 };
 struct Pass {                                      // one pass through the layers
     Ctx & c; Stack & st; hipStream_t s; bamd_batch_dev b; bool decode = false;
-    int n_tiles = 0, k_rows = 0, max_n = 1; float * x; float * xo; const float * pend = nullptr; int ldp = 0; const float * pend_g = nullptr;
+    int n_tiles = 0, k_rows = 0, max_n = 1, n_segs = 0; float * x; float * xo; const float * pend = nullptr; int ldp = 0; const float * pend_g = nullptr;
     Timer * tm = nullptr;
     void begin(int kind, double bytes) { if (!tm) return; hipEvent_t e; hipEventCreate(&e); hipEventRecord(e, s); tm->ev.push_back(e); tm->kind.push_back(kind); tm->bytes.push_back(bytes); }
     void end() { if (!tm) return; hipEvent_t e; hipEventCreate(&e); hipEventRecord(e, s); tm->ev.push_back(e); }
 
-    bamd_residual_args residual(const float * mu, float * prev) {
+    bamd_residual_args residual(const float * mu, float * prev, const float * gi) {
         bamd_residual_args a; memset(&a, 0, sizeof a);
+        a.norm = st.d.norm == STACK_NORM_SANDWICH ? BAMD_NORM_LAYER : BAMD_NORM_RMS; a.gi = gi;
         a.x = x; a.y = pend; a.ldy = ldp; a.g = pend_g; a.eps = st.eps; a.mu = mu; a.prev = prev; a.xo = xo; a.h = c.h; a.E = st.E; a.ldh = up(st.E, 32);
         return a;
     }
@@ -214,6 +233,7 @@ struct Pass {                                      // one pass through the layer
         begin(2, 0);
         int ldx = 0;
         if (pre == BAMD_PRE_RESIDUAL) { bamd_launch_residual_rows(st.act, b, p.res, s); ldx = p.res.ldh; }
+        else if (pre == BAMD_PRE_GLU) { bamd_launch_glu_rows(st.act, b.rows, p.glu, s); ldx = p.glu.ldh; }
         else if (pre == BAMD_PRE_POLY) { bamd_launch_poly_rows(st.act, b.rows, p.poly, s); ldx = p.poly.ldh; }
         else { bamd_launch_group_norm_rows(st.act, b.rows, p.grp, s); ldx = p.grp.ldh; }
         end();
@@ -275,15 +295,169 @@ struct LatentAttention : Mixer {
         return l.vec(p + "dkv.norm", { R }, &c_norm) || (dz.latent_sink && l.vec(p + "sink", { H }, &sink));
     }
     int latents() const override { return Rp; }
+    int prompt_rows(int act) const override { return bamd_latent_prompt_rows(act, D); }
     double step_bytes(int len) const override { return (double) len * R * 2; }
     int state(Ctx & c, MixState & st) override;
     int run(Pass & p, MixState & st, Operand & o) override;
+};
+// ---- branches: mixers that share one input projection and one output projection (their results are summed there) ------------------------------------------
+struct Part { const SafeTensor * t; std::vector<int32_t> rows, cols; int at; };       // of a packed matrix, at its row / column `at`
+struct Branch {
+    int in0 = 0, in_rows = 0, out0 = 0, out_cols = 0; float out_scale = 1;            // rows of the input projection, columns of the output projection
+    virtual ~Branch() {}
+    // in0, out0, out_scale are set; sets in_rows (a multiple of 16) and out_cols (of 32)
+    virtual int load(Loader & l, const Conf & c, const std::string & p, int E, float eps, const bamd_stack_design & d, std::vector<Part> & in, std::vector<Part> & out) = 0;
+    virtual int state(Ctx & c, MixState & st) = 0;
+    virtual int run(Pass & p, MixState & st, int ld, int ldo) = 0;                    // p.c.y: rows of the input projection -> p.c.h: operand of the output projection
+    virtual double step_bytes(int len) const = 0;
+    virtual int f32_cols() const { return 0; }
+    virtual int prompt_rows(int) const { return 0; }
+    virtual int scan_blocks() const { return 0; }
+    virtual void partials(int, size_t &, size_t &) const {}
+};
+// the bias of every distance up to `top` (and everything farther) from a table [rows][heads]: one row per distance in the first half, logarithmic steps in the second
+std::vector<float> expand_bias(const std::vector<float> & rel, int rows, int heads, int top) {
+    std::vector<float> h((size_t) heads * (top + 1));
+    const int half = rows / 2;
+    for (int n = 0; n <= top; ++n) {
+        // (a step that falls on a whole distance belongs to it, whatever the logarithms round to)
+        const int k = n < half ? n : std::min(rows - 1, half + (int) floor(log((double) n / half) / log((double) top / half) * (rows - half) + 1e-9));
+        for (int i = 0; i < heads; ++i) h[(size_t) i * (top + 1) + n] = rel[(size_t) k * heads + i];
+    }
+    return h;
+}
+int kv_splits(const bamd_kv_args & a, int rows, int max_pages) {
+    const int groups = std::max(1, rows * bamd_kv_groups(a)), span = bamd_kv_span(a, max_pages);
+    return std::max(1, std::min({ (span + 1 + 3) / 4, std::max(1, 1024 / groups), 64 }));        // four waves per share, the row's own key is one more page
+}
+struct KvAttention : Branch {
+    bamd_kv_args a; int vdim = 0;
+    KvAttention() { memset((void *) &a, 0, sizeof a); }
+    int load(Loader & l, const Conf & c, const std::string & p, int E, float eps, const bamd_stack_design & d, std::vector<Part> & in, std::vector<Part> & out) override {
+        int H, G;
+        if (c.size("heads", H) || c.size("kv_heads", G) || c.size("dim", a.dim, 1, 256) || c.size("vdim", vdim, 1, 256) || c.f32("scale", a.scale) || (d.kv_cap && c.f32("softcap", a.cap))) return 1;
+        if (H % G) return fail("config.json: " + c.where + "heads is no multiple of kv_heads");
+        if (d.kv_cap && !(a.cap > 0)) return fail("config.json: " + c.where + "softcap out of range");
+        a.heads = H; a.kv_heads = G; a.eps = eps; a.unit = d.kv_unit; a.gated = d.kv_gate; a.out_scale = out_scale; a.out_off = out0;
+        a.window = 0x3fffffff; a.keep = 0;
+        const Json * mask = c.j->get("mask");
+        if (mask && mask->kind == Json::OBJ) {
+            const Conf mc{ mask, c.where + "mask." };
+            if (mc.size("size", a.window) || mc.size("keep_first", a.keep, 0)) return 1;
+        }
+        for (a.D = 32; a.D < std::max(a.dim, vdim); a.D *= 2) {}
+        const int D = a.D;
+        if (d.kv_bias) {
+            const int B = l.dim(p + "rel", 0);
+            std::vector<float> rel; float * dev;
+            if (c.size("bias_max", a.bias_top, 1, 1 << 24) || l.values(p + "rel", { B, H }, rel)) return 1;
+            if (a.bias_top <= B / 2 || B < 2) return fail("config.json: " + c.where + "bias_max is not above half of the bias table's rows");
+            if (l.upload(expand_bias(rel, B, H, a.bias_top), &dev)) return 1;
+            a.bias = dev;
+        }
+        // [q, each head padded to D | k | v | gates]
+        const SafeTensor * tq = l.matrix(p + "q", { H * a.dim, E }), * tk = l.matrix(p + "k", { G * a.dim, E }), * tv = l.matrix(p + "v", { G * vdim, E }), * to = l.matrix(p + "o", { E, H * vdim });
+        const SafeTensor * tg = d.kv_gate ? l.matrix(p + "g", { H, E }) : nullptr;
+        if (!tq || !tk || !tv || !to || (d.kv_gate && !tg)) return 1;
+        const std::vector<int32_t> cols = Loader::steps(E, 1);
+        a.q_off = in0; a.k_off = a.q_off + H * D; a.v_off = a.k_off + G * D; a.g_off = a.v_off + G * D;
+        in.push_back({ tq, Loader::grouped(H, a.dim, D, E), cols, a.q_off }); in.push_back({ tk, Loader::grouped(G, a.dim, D, E), cols, a.k_off }); in.push_back({ tv, Loader::grouped(G, vdim, D, E), cols, a.v_off });
+        if (tg) in.push_back({ tg, Loader::steps(H, E), cols, a.g_off });
+        out.push_back({ to, Loader::steps(E, H * vdim), Loader::grouped(H, vdim, D, 1), out0 });
+        in_rows = a.g_off + (tg ? up(H, 16) : 0) - in0; out_cols = H * D;
+        return 0;
+    }
+    double step_bytes(int len) const override { return (double) std::min<long>(len, (long) a.window + a.keep) * a.kv_heads * (a.dim + vdim) * 2; }
+    int prompt_rows(int act) const override { return bamd_kv_prompt_rows(act, a.D); }
+    void partials(int rows, size_t & po, size_t & pm) const override {
+        const size_t cells = std::max<size_t>(1024, (size_t) rows * bamd_kv_groups(a));       // rows x groups x splits never exceeds this (kv_splits)
+        po = std::max(po, cells * 16 * a.D); pm = std::max(pm, cells * 32);
+    }
+    int state(Ctx & c, MixState & st) override;
+    int run(Pass & p, MixState & st, int ld, int ldo) override;
+};
+struct GatedLinear : Branch {
+    bamd_gla_args a; int N = 0;
+    GatedLinear() { memset((void *) &a, 0, sizeof a); }
+    int load(Loader & l, const Conf & c, const std::string & p, int E, float eps, const bamd_stack_design & d, std::vector<Part> & in, std::vector<Part> & out) override {
+        int H; float tau;
+        if (c.size("heads", H) || c.size("dim", N, 1, 256) || c.size("vdim", a.P) || c.f32("tau", tau)) return 1;
+        if (!(tau > 0)) return fail("config.json: " + c.where + "tau out of range");
+        const int P = a.P, R = l.dim(p + "a1", 0);
+        if (R > 1024) return fail("tensor " + p + "a1: rank above 1024");
+        a.heads = H; a.Np = up(N, 4); a.Pp = up(P, 4); a.rank = R; a.inv_tau = 1.f / tau; a.q_scale = (float) (1.0 / sqrt((double) N)); a.eps = eps; a.out_off = out0;
+        const SafeTensor * tq = l.matrix(p + "q", { H * N, E }), * tk = l.matrix(p + "k", { H * N, E }), * tv = l.matrix(p + "v", { H * P, E }), * tg = d.gla_gate ? l.matrix(p + "g", { H * P, E }) : nullptr;
+        const SafeTensor * t1 = l.matrix(p + "a1", { R, E }), * t2 = l.matrix(p + "a2", { H * N, R }), * to = l.matrix(p + "o", { E, H * P });
+        if (!tq || !tk || !tv || (d.gla_gate && !tg) || !t1 || !t2 || !to) return 1;
+        // [q | k | v | gate, heads padded to four | the decays' low rank]
+        const std::vector<int32_t> cols = Loader::steps(E, 1);
+        a.q_off = in0; a.k_off = a.q_off + up(H * a.Np, 16); a.v_off = a.k_off + up(H * a.Np, 16); a.g_off = a.v_off + up(H * a.Pp, 16); a.t_off = a.g_off + (tg ? up(H * a.Pp, 16) : 0);
+        in.push_back({ tq, Loader::grouped(H, N, a.Np, E), cols, a.q_off }); in.push_back({ tk, Loader::grouped(H, N, a.Np, E), cols, a.k_off }); in.push_back({ tv, Loader::grouped(H, P, a.Pp, E), cols, a.v_off });
+        if (tg) in.push_back({ tg, Loader::grouped(H, P, a.Pp, E), cols, a.g_off }); else a.g_off = -1;
+        in.push_back({ t1, Loader::steps(R, E), cols, a.t_off });
+        in_rows = a.t_off + up(R, 16) - in0; out_cols = up(H * a.Pp, 32);
+        a.out_cols = out_cols;
+        std::vector<int32_t> oc = Loader::grouped(H, P, a.Pp, 1); oc.resize((size_t) out_cols, -1);
+        out.push_back({ to, Loader::steps(E, H * P), oc, out0 });
+        // second factor of the decays, transposed: neighbouring channels are neighbours
+        std::vector<uint16_t> w((size_t) R * H * a.Np, 0); std::vector<float> bias, pb((size_t) H * a.Np, 0.f), nm;
+        for (int i = 0; i < H * N; ++i) for (int r = 0; r < R; ++r) memcpy(&w[(size_t) r * H * a.Np + (size_t) (i / N) * a.Np + i % N], t2->data + ((size_t) i * R + r) * 2, 2);
+        if (l.values(p + "a2.b", { H * N }, bias) || l.values(p + "norm", { P }, nm)) return 1;
+        for (int i = 0; i < H * N; ++i) pb[(size_t) (i / N) * a.Np + i % N] = bias[(size_t) i];
+        for (float & v : nm) v *= out_scale;
+        nm.resize((size_t) a.Pp, 0.f);
+        uint16_t * dw; float * db, * dn;
+        if (l.upload(w, &dw) || l.upload(pb, &db) || l.upload(nm, &dn)) return 1;
+        a.a2 = dw; a.a2b = db; a.norm = dn;
+        l.m->weight_bytes += (int64_t) t2->nbytes;
+        return 0;
+    }
+    double step_bytes(int) const override { return 8.0 * a.heads * N * a.P; }
+    int f32_cols() const override { return a.heads * a.Pp; }
+    int scan_blocks() const override { return bamd_gla_blocks(a.heads, a.Pp); }
+    int state(Ctx & c, MixState & st) override;
+    int run(Pass & p, MixState & st, int ld, int ldo) override;
+};
+// several branches over one input, their outputs summed with a scale each
+struct Parallel : Mixer {
+    std::vector<std::unique_ptr<Branch>> br;
+    int load(Loader & l, const Conf & c, const std::string & p, int E, float eps, const bamd_stack_design & d) override {
+        std::vector<Part> pi, po;
+        const char * sides[2] = { "left", "right" };
+        br.emplace_back(new KvAttention()); br.emplace_back(new GatedLinear());
+        int ni = 0, no = 0;
+        for (int i = 0; i < 2; ++i) {
+            const std::string side = sides[i];
+            Branch & b = *br[(size_t) i];
+            const Json * j = c.j ? c.j->get(side) : nullptr;
+            if (!j || j->kind != Json::OBJ) return fail("config.json: " + c.where + side + " missing");
+            b.in0 = ni; b.out0 = no;
+            if (c.f32((side + "_scale").c_str(), b.out_scale) || b.load(l, Conf{ j, c.where + side + "." }, p + side + ".", E, eps, d, pi, po)) return 1;
+            ni += b.in_rows; no += b.out_cols;
+        }
+        if (l.alloc(in, ni, E) || l.alloc(out, E, no)) return 1;
+        for (const Part & q : pi) if (l.pack(q.t, q.rows, q.cols, const_cast<uint16_t *>(in.w) + (size_t) q.at * in.K)) return 1;
+        for (const Part & q : po) if (l.pack(q.t, q.rows, q.cols, const_cast<uint16_t *>(out.w) + (size_t) (q.at / 32) * 512, 1, out.k_tiles)) return 1;
+        return 0;
+    }
+    int state(Ctx & c, MixState & st) override {
+        st.sub.resize(br.size());
+        for (size_t i = 0; i < br.size(); ++i) if (br[i]->state(c, st.sub[i])) return 1;
+        return 0;
+    }
+    int run(Pass & p, MixState & st, Operand & o) override;
+    double step_bytes(int len) const override { double t = 0; for (auto & b : br) t += b->step_bytes(len); return t; }
+    int f32_cols() const override { int n = 0; for (auto & b : br) n = std::max(n, b->f32_cols()); return n; }
+    int prompt_rows(int act) const override { int n = 0; for (auto & b : br) if (const int q = b->prompt_rows(act)) n = n ? std::min(n, q) : q; return n; }
+    int scan_blocks() const override { int n = 0; for (auto & b : br) n = std::max(n, b->scan_blocks()); return n; }
+    void partials(int rows, size_t & po, size_t & pm) const override { for (auto & b : br) b->partials(rows, po, pm); }
 };
 std::unique_ptr<Mixer> make_mixer(const std::string & type, const bamd_stack_design & d) {
     const std::string all = std::string(" ") + d.mixers + " ";
     if (all.find(" " + type + " ") == std::string::npos) return nullptr;
     if (type == "mamba2") return std::unique_ptr<Mixer>(new Mamba2());
     if (type == "latent_attention") return std::unique_ptr<Mixer>(new LatentAttention());
+    if (type == "parallel") return std::unique_ptr<Mixer>(new Parallel());
     return nullptr;
 }
 
@@ -296,7 +470,7 @@ int Stack::load(bamd_model * model, const bamd_load_args & a, const bamd_stack_d
     if (!Json::parse(text.data(), text.data() + text.size(), j, err)) return fail(dir + "/config.json: " + err);
     const Conf top{ &j, "" };
     const Json * ls = j.get("layers");
-    if (top.size("vocab", V) || top.size("width", E) || Conf{ j.get("embedding"), "embedding." }.f32("scale", scale) || Conf{ j.get("norm"), "norm." }.f32("eps", eps)) return 1;
+    if (top.size("vocab", V) || top.size("width", E) || (d.scaled_embedding && Conf{ j.get("embedding"), "embedding." }.f32("scale", scale)) || Conf{ j.get("norm"), "norm." }.f32("eps", eps)) return 1;
     if (d.learned_positions && top.size("max_positions", max_pos)) return 1;
     if (!ls || ls->kind != Json::ARR || ls->arr.empty()) return fail("config.json: layers missing");
     L = (int) ls->arr.size();
@@ -318,7 +492,11 @@ int Stack::load(bamd_model * model, const bamd_load_args & a, const bamd_stack_d
     { hipDeviceProp_t p; HIPC(hipGetDeviceProperties(&p, a.device)); m->n_cu = p.multiProcessorCount > 0 ? p.multiProcessorCount : 256; }
     HIPC(hipStreamCreate(&l.s));
     if (m->with_embd && (l.raw("embed", { V, E }, &embd) || (d.learned_positions && l.raw("pos", { max_pos, E }, &pos)))) return 1;
-    if (m->with_output && (l.vec("final.norm", {}, &norm_f) || l.plain("head", V, E, head))) return 1;
+    const bool sandwich = d.norm == STACK_NORM_SANDWICH;
+    const std::vector<int64_t> gain = sandwich ? std::vector<int64_t>{ E } : std::vector<int64_t>{};      // shape of a norm's gain
+    float logit_scale = 1.f;                                     // enters with the last norm's gain
+    if (d.tied_head && top.f32("logit_scale", logit_scale)) return 1;
+    if (m->with_output && (l.vec("final.norm", gain, &norm_f, logit_scale) || l.plain(d.tied_head ? "embed" : "head", V, E, head))) return 1;
     layers.resize((size_t) (ll - lf));
     for (int il = lf; il < ll; ++il) {
         Layer & ly = layers[(size_t) (il - lf)];
@@ -329,13 +507,23 @@ int Stack::load(bamd_model * model, const bamd_load_args & a, const bamd_stack_d
         ly.mix = make_mixer(type->str, d);
         if (!ly.mix) return fail("config.json: " + where + "type \"" + type->str + "\" is not one of this architecture's mixers (" + d.mixers + ")");
         if (ly.mix->load(l, Conf{ cj.get("mixer"), where + "mixer." }, p + "mix.", E, eps, d)) return 1;
-        if (l.vec(p + "norm1", {}, &ly.norm1) || (d.token_shift && l.vec(p + "shift", { E }, &ly.shift))) return 1;
+        if (sandwich ? l.vec(p + "norm1", gain, &ly.pre1) || l.vec(p + "norm1b", gain, &ly.norm1, 1.f, p + "ls1") : l.vec(p + "norm1", gain, &ly.norm1)) return 1;
+        if ((d.token_shift && l.vec(p + "shift", { E }, &ly.shift))) return 1;
         ly.mlp = mlp && mlp->kind == Json::OBJ;
         if (ly.mlp) {
             const Json * kind = mlp->get("kind");
             if (!kind || kind->str != "dense") return fail("config.json: " + where + "mlp.kind is not \"dense\"");
             if (Conf{ mlp, where + "mlp." }.size("ff", ly.F)) return 1;
-            if (l.plain(p + "mlp.up", ly.F, E, ly.up) || l.plain(p + "mlp.down", E, ly.F, ly.down) || l.vec(p + "mlp.act", { 4 }, &ly.act) || l.vec(p + "norm2", {}, &ly.norm2)) return 1;
+            if (sandwich ? l.vec(p + "norm2", gain, &ly.pre2) || l.vec(p + "norm2b", gain, &ly.norm2, 1.f, p + "ls2") : l.vec(p + "norm2", gain, &ly.norm2)) return 1;
+            if (l.plain(p + "mlp.down", E, ly.F, ly.down)) return 1;
+            if (d.mlp_act == STACK_ACT_CLAMPED_GLU) {
+                // gate and up rows in turn, sixteen of each: one wave holds both halves of its outputs
+                const SafeTensor * tg = l.matrix(p + "mlp.gate", { ly.F, E }), * tu = l.matrix(p + "mlp.up", { ly.F, E });
+                if (!tg || !tu || Conf{ mlp, where + "mlp." }.f32("limit", ly.limit) || l.alloc(ly.up, 2 * ly.down.K, E)) return 1;
+                std::vector<int32_t> rows = Loader::steps(ly.F, E); rows.resize((size_t) ly.down.K, -1);
+                uint16_t * w = const_cast<uint16_t *>(ly.up.w);
+                if (l.pack(tg, rows, Loader::steps(E, 1), w, 2) || l.pack(tu, rows, Loader::steps(E, 1), w + (size_t) 16 * ly.up.K, 2)) return 1;
+            } else if (l.plain(p + "mlp.up", ly.F, E, ly.up) || l.vec(p + "mlp.act", { 4 }, &ly.act)) return 1;
         }
     }
     return 0;
@@ -350,6 +538,11 @@ int LatentAttention::state(Ctx & c, MixState & st) {
     const size_t n_pages = c.free_pages.size();
     return dev_alloc(c.c->allocs, &st.cache, n_pages * BAMD_PAGE * Rp * c.st->el());
 }
+int KvAttention::state(Ctx & c, MixState & st) {
+    const size_t n = (size_t) c.free_pages.size() * a.kv_heads * BAMD_PAGE * a.D * c.st->el();
+    return dev_alloc(c.c->allocs, &st.cache, n) || dev_alloc(c.c->allocs, &st.cache2, n);
+}
+int GatedLinear::state(Ctx & c, MixState & st) { return dev_alloc(c.c->allocs, (void **) &st.b, (size_t) c.c->n_seq * a.heads * a.Np * a.Pp * 4); }
 Ctx & ctx_of(bamd_context * c) { return *(Ctx *) c->arch_state; }
 
 int Stack::context_init(bamd_context * bc) {
@@ -374,11 +567,13 @@ int Stack::context_init(bamd_context * bc) {
             const size_t hg = (size_t) (la->H + 15) / 16, cells = 512 + (size_t) brows * hg;     // rows x head groups x splits never exceeds this (splits_for)
             qp = std::max(qp, (size_t) brows * hg * 16 * la->Rp); po = std::max(po, cells * 16 * la->Rp); pm = std::max(pm, cells * 32);
         }
+        mx.partials(brows, po, pm);
     }
     const size_t R = (size_t) c.rows_cap;
     if (dev_alloc(bc->allocs, (void **) &c.xa, R * E * 4) || dev_alloc(bc->allocs, (void **) &c.xb, R * E * 4) || dev_alloc(bc->allocs, (void **) &c.y, R * std::max(c.ldy, 16) * 4) ||
         dev_alloc(bc->allocs, (void **) &c.y2, R * c.ldy2 * 4) || dev_alloc(bc->allocs, (void **) &c.y3, R * std::max(c.ldy3, 16) * 4) || dev_alloc(bc->allocs, &c.h, R * c.ldh * el())) return 1;
-    if (qp && (dev_alloc(bc->allocs, &c.qp, qp * el()) || dev_alloc(bc->allocs, (void **) &c.part_o, po * 4) || dev_alloc(bc->allocs, (void **) &c.part_ml, pm * 4))) return 1;
+    if (qp && dev_alloc(bc->allocs, &c.qp, qp * el())) return 1;
+    if (po && (dev_alloc(bc->allocs, (void **) &c.part_o, po * 4) || dev_alloc(bc->allocs, (void **) &c.part_ml, pm * 4))) return 1;
     if (qp) HIPC(hipMemset(c.qp, 0, qp * el()));                  // rows of absent heads stay zero
     c.mix.resize(layers.size()); c.prev.resize(layers.size());
     for (size_t i = 0; i < layers.size(); ++i) {
@@ -389,10 +584,10 @@ int Stack::context_init(bamd_context * bc) {
     if (dev_alloc(bc->allocs, (void **) &c.keys, std::max<size_t>((size_t) S, BAMD_LOGIT_ROWS) * 8) || dev_alloc(bc->allocs, (void **) &c.step, 4) || dev_alloc(bc->allocs, (void **) &c.gen_out, (size_t) S * c.gen_cap * 4)) return 1;
     Ctx::Layout & y = c.lay;
     const int max_e = S;
-    y.tiles = (int) R / 16 + max_e; y.kblks = c.max_pages + S;
+    y.tiles = (int) R / 16 + max_e; y.kblks = c.max_pages + S; y.segs = (int) R / SEG_MIN + max_e;
     size_t at = 0;
     auto put = [&](size_t bytes) { const size_t p = at; at = (at + bytes + 63) / 64 * 64; return p; };
-    y.ent = put(sizeof(bamd_entry) * (size_t) max_e); y.row = put(R * 4); y.tok = put(R * 4); y.want = put(R * 4); y.tile = put(sizeof(bamd_qtile) * (size_t) y.tiles); y.kblk = put((size_t) y.kblks * 4);
+    y.ent = put(sizeof(bamd_entry) * (size_t) max_e); y.row = put(R * 4); y.tok = put(R * 4); y.want = put(R * 4); y.tile = put(sizeof(bamd_qtile) * (size_t) y.tiles); y.kblk = put((size_t) y.kblks * 4); y.seg = put(sizeof(bamd_segment) * (size_t) y.segs);
     y.total = at;
     if (dev_alloc(bc->allocs, (void **) &c.dev, y.total) || dev_alloc(bc->allocs, (void **) &c.pages, (size_t) S * c.max_pages * 4)) return 1;
     for (int i = 0; i < Ctx::RING; ++i) {
@@ -406,7 +601,7 @@ void Stack::context_free(bamd_context * bc) {
     if (!c) return;
     for (auto & g : c->graphs) hipGraphExecDestroy(g.second);
     for (int i = 0; i < Ctx::RING; ++i) { if (c->host[i]) hipHostFree(c->host[i]); if (c->pages_host[i]) hipHostFree(c->pages_host[i]); if (c->ev[i]) hipEventDestroy(c->ev[i]); }
-    for (void * p : { c->kc, c->kk, c->kv, (void *) c->filtered, (void *) c->steps }) if (p) hipFree(p);
+    for (void * p : { c->kc, c->kk, c->kv, (void *) c->filtered, (void *) c->steps, (void *) c->alpha, (void *) c->seg_state, (void *) c->seg_decay }) if (p) hipFree(p);
     delete c;
     bc->arch_state = nullptr;
 }
@@ -474,12 +669,46 @@ int LatentAttention::run(Pass & p, MixState & st, Operand & o) {
     p.end();
     return rc ? fail("latent attention: unsupported shape") : 0;
 }
+int KvAttention::run(Pass & p, MixState & st, int ld, int ldo) {
+    Ctx & c = p.c;
+    const int act = p.st.act;
+    bamd_kv_args k = a;
+    k.in = c.y; k.ld = ld; k.kc = st.cache; k.vc = st.cache2; k.out = c.h; k.ldo = ldo;
+    int rc = 0;
+    if (p.decode) rc = bamd_launch_kv_decode(act, p.b, k, c.part_o, c.part_ml, kv_splits(k, p.b.rows, c.max_pages), p.s);
+    else {
+        bamd_launch_kv_store(act, p.b, k, (const int32_t *) (c.dev + c.lay.kblk), p.k_rows, p.s);
+        rc = bamd_launch_kv_prompt(act, p.b, k, (const bamd_qtile *) (c.dev + c.lay.tile), p.n_tiles, p.s);
+    }
+    return rc ? fail("attention over keys and values: unsupported shape") : 0;
+}
+int GatedLinear::run(Pass & p, MixState & st, int ld, int ldo) {
+    Ctx & c = p.c;
+    bamd_gla_args g = a;
+    g.in = c.y; g.ld = ld; g.state = st.b; g.y = c.y3; g.ldy = a.heads * a.Pp; g.out = c.h; g.ldo = ldo;
+    if (p.max_n > 1) {
+        const size_t ch = (size_t) a.heads * a.Np;
+        if (grow(c, (void **) &c.alpha, &c.alpha_n, (size_t) p.b.rows * ch * 4, p.s)) return 1;
+        if (p.n_segs > p.b.n_entries && (grow(c, (void **) &c.seg_state, &c.seg_state_n, p.n_segs * ch * a.Pp * 4, p.s) || grow(c, (void **) &c.seg_decay, &c.seg_decay_n, p.n_segs * ch * 4, p.s))) return 1;
+        g.alpha = c.alpha; g.seg_state = c.seg_state; g.seg_decay = c.seg_decay;
+    }
+    if (bamd_launch_gla(p.b, g, p.max_n, (const bamd_segment *) (c.dev + c.lay.seg), p.n_segs, p.s)) return fail("gated linear attention: unsupported shape");
+    bamd_launch_gla_norm(p.st.act, g, p.b.rows, p.s);
+    return 0;
+}
+int Parallel::run(Pass & p, MixState & st, Operand & o) {
+    o.x = p.c.h; o.ldx = out.K;
+    p.begin(1, p.tm ? step_bytes(p.c.seqs[0].len + 1) : 0);
+    for (size_t i = 0; i < br.size(); ++i) if (br[i]->run(p, st.sub[i], ld_of(in), out.K)) return 1;
+    p.end();
+    return 0;
+}
 int Pass::layers() {
     bamd_pre_args pa; memset((void *) &pa, 0, sizeof pa);
     for (size_t i = 0; i < st.layers.size(); ++i) {
         Layer & ly = st.layers[i];
         Mixer & mx = *ly.mix;
-        pa.res = residual(ly.shift, c.prev[i]);
+        pa.res = residual(ly.shift, c.prev[i], ly.pre1);
         if (product_pre(mx.in, BAMD_PRE_RESIDUAL, pa, c.y, ld_of(mx.in), 0)) return 1;
         Operand o;
         if (mx.run(*this, c.mix[i], o)) return 1;
@@ -487,16 +716,27 @@ int Pass::layers() {
         else { pa.grp = o.grp; if (product_pre(mx.out, o.pre, pa, c.y2, c.ldy2, 3)) return 1; }
         advanced(c.y2, c.ldy2, ly.norm1);
         if (!ly.mlp) continue;
-        pa.res = residual(nullptr, nullptr);
-        if (product_pre(ly.up, BAMD_PRE_RESIDUAL, pa, c.y, ld_of(ly.up), 4)) return 1;
-        pa.poly = { c.y, ld_of(ly.up), ly.act, st.eps, c.h, ly.F, ly.down.K };
-        if (product_pre(ly.down, BAMD_PRE_POLY, pa, c.y2, c.ldy2, 5)) return 1;
+        pa.res = residual(nullptr, nullptr, ly.pre2);
+        const bool glu = st.d.mlp_act == STACK_ACT_CLAMPED_GLU;
+        if (glu && b.rows > BAMD_MV_ROWS) {                        // the product's tiles write the down-projection's operand
+            begin(2, 0); bamd_launch_residual_rows(st.act, b, pa.res, s); end();
+            begin(4, (double) ly.up.bytes);
+            const int rc = bamd_launch_dense_gemm(st.act, ly.up, c.h, pa.res.ldh, b.rows, c.y, ly.down.K, BAMD_OUT_GLU, s, ly.limit);
+            end();
+            if (rc) return fail("dense product: unsupported shape");
+            if (product(ly.down, c.y, ly.down.K, c.y2, c.ldy2, 5)) return 1;
+        } else {
+            if (product_pre(ly.up, BAMD_PRE_RESIDUAL, pa, c.y, ld_of(ly.up), 4)) return 1;
+            if (glu) pa.glu = { c.y, ld_of(ly.up), ly.limit, c.h, ly.down.K };
+            else pa.poly = { c.y, ld_of(ly.up), ly.act, st.eps, c.h, ly.F, ly.down.K };
+            if (product_pre(ly.down, glu ? BAMD_PRE_GLU : BAMD_PRE_POLY, pa, c.y2, c.ldy2, 5)) return 1;
+        }
         advanced(c.y2, c.ldy2, ly.norm2);
     }
     return 0;
 }
 int Pass::head(const int32_t * want, int n, float * logits) {
-    bamd_residual_args a = residual(nullptr, nullptr);
+    bamd_residual_args a = residual(nullptr, nullptr, nullptr);
     if (fused(st.head) && n == 1) {
         bamd_pre_args pa; memset((void *) &pa, 0, sizeof pa);
         pa.res = a; pa.gf = st.norm_f; pa.want = want;
@@ -525,7 +765,11 @@ int send(Pass & p, const std::vector<Piece> & pc, const std::vector<int32_t> & w
     int32_t * row = (int32_t *) (h + c.lay.row), * tok = (int32_t *) (h + c.lay.tok), * kblk = (int32_t *) (h + c.lay.kblk);
     bamd_qtile * tile = (bamd_qtile *) (h + c.lay.tile);
     int rows = 0, kb = 0, nt = 0, tq = 0;
-    for (const Layer & ly : p.st.layers) if (auto * la = dynamic_cast<LatentAttention *>(ly.mix.get())) { const int q = bamd_latent_prompt_rows(p.st.act, la->D); tq = tq ? std::min(tq, q) : q; }
+    int scan = 0;
+    for (const Layer & ly : p.st.layers) {
+        if (const int q = ly.mix->prompt_rows(p.st.act)) tq = tq ? std::min(tq, q) : q;
+        scan = std::max(scan, ly.mix->scan_blocks());
+    }
     for (size_t e = 0; e < pc.size(); ++e) {
         Seq & q = c.seqs[(size_t) pc[e].seq];
         ent[e] = { pc[e].seq, rows, pc[e].n, q.len, q.par, kb * BAMD_PAGE };
@@ -542,6 +786,17 @@ int send(Pass & p, const std::vector<Piece> & pc, const std::vector<int32_t> & w
         for (size_t e = 0; e < pc.size(); ++e) for (int q0 = 0; q0 < pc[e].n; q0 += tq) tile[nt++] = { (int32_t) e, q0 };
         std::stable_sort(tile, tile + nt, [&](const bamd_qtile & a, const bamd_qtile & b) { return ent[a.entry].pos0 + a.q0 > ent[b.entry].pos0 + b.q0; });
     }
+    // scan segments: as many as fill the chip, none short
+    int ns = 0;
+    if (!p.decode && scan) {
+        const int shortest = std::max(SEG_MIN, (rows + (SEG_BLOCKS + scan - 1) / scan - 1) / ((SEG_BLOCKS + scan - 1) / scan));
+        bamd_segment * seg = (bamd_segment *) (h + c.lay.seg);
+        for (size_t e = 0; e < pc.size(); ++e) {
+            const int n = pc[e].n, k = std::max(1, std::min(n / shortest, n / (2 * SEG_MIN))), len = up((n + k - 1) / k, 8), first = ns;
+            for (int t = 0; t < n; t += len) seg[ns++] = { (int32_t) e, t, std::min(len, n - t), first, 0 };
+            for (int i = first; i < ns; ++i) seg[i].last = ns - 1;
+        }
+    }
     memcpy(h + c.lay.want, want.data(), want.size() * 4);
     HIPC(hipMemcpyAsync(c.dev, h, c.lay.total, hipMemcpyHostToDevice, p.s));
     if (c.pages_dirty) {
@@ -551,7 +806,7 @@ int send(Pass & p, const std::vector<Piece> & pc, const std::vector<int32_t> & w
     }
     HIPC(hipEventRecord(c.ev[r], p.s));
     p.b = { (bamd_entry *) (c.dev + c.lay.ent), (int32_t *) (c.dev + c.lay.row), (int32_t *) (c.dev + c.lay.tok), (int) pc.size(), rows, c.c->n_seq, c.pages, c.max_pages };
-    p.k_rows = kb * BAMD_PAGE; p.n_tiles = nt;
+    p.k_rows = kb * BAMD_PAGE; p.n_tiles = nt; p.n_segs = ns;
     p.x = c.xa; p.xo = c.xb; p.pend = nullptr; p.ldp = 0; p.pend_g = nullptr;
     return 0;
 }
@@ -720,7 +975,7 @@ int Stack::stage(bamd_context * bc, const int32_t * tokens, const void * token_d
     if (p.layers()) return 1;
     moved(c, pc);
     if (!m->with_output) {
-        bamd_residual_args a = p.residual(nullptr, nullptr);
+        bamd_residual_args a = p.residual(nullptr, nullptr, nullptr);
         a.xo = (float *) hout; a.h = nullptr;
         bamd_launch_residual_rows(act, p.b, a, s);
     } else if (want_logits) {
