@@ -211,7 +211,7 @@ def main():
     ap.add_argument("--backend", default="nccl", choices=["nccl", "gloo"], help="gloo: CPU plumbing check of the N > 1 leg (launch, rendezvous, schedule, JSON) "
                                                                                "with a stand-in stage — tests/test_bench_selflaunch.py; never a measurement")
     ap.add_argument("--no-secondary", action="store_true", help="skip the secondary configurations (BASELINE configs 3, 5 and 4 at N = 1) of the N = 1 line")
-    ap.add_argument("--stack", action="store_true", help="instead: configured layer stacks (Tupitar: latent attention + Mamba-2, bfloat16) beside Llama Q4_K_M at equal layer sizes, "
+    ap.add_argument("--stack", action="store_true", help="instead: configured layer stacks (Tupitar: latent attention + Mamba-2; Mafurax: windowed attention beside gated linear attention; bfloat16) beside Llama Q4_K_M at equal layer sizes, "
                                                           "prompt and decode throughput and per-launch-kind rates, one JSON line")
     args = ap.parse_args()
     if args.stack:
@@ -577,16 +577,19 @@ def bridge_longctx_rate(n_pos=7900):
 STACK_KINDS = ["in_projection", "mixer", "other", "out_projection", "mlp_up", "mlp_down", "lm_head"]
 
 
-def stack_config(E, F, H, hd, R, mheads, P, state, L, V=32000, max_positions=8192):
-    """L layers, latent attention and Mamba-2 in turn, at the sizes of a real model's layers"""
+def stack_configs(E, F, H, hd, R, mheads, P, state, gheads, gdim, gvdim, window, L, V=32000, max_positions=8192):
+    """L layers at the sizes of a real model's layers: Tupitar (latent attention and Mamba-2 in turn) and Mafurax (windowed attention and gated linear attention side by side)"""
     mlp = {"kind": "dense", "ff": F}
     at = {"type": "latent_attention", "mixer": dict(heads=H, dim=hd, vdim=hd, kv_rank=R, scale=hd ** -0.5), "mlp": mlp}
     mb = {"type": "mamba2", "mixer": dict(heads=mheads, vdim=P, state=state, groups=1, norm_groups=1, conv=4), "mlp": mlp}
-    return {"architecture": "Tupitar", "vocab": V, "width": E, "max_positions": max_positions, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6}, "layers": [at, mb] * (L // 2)}
+    left = dict(heads=H, kv_heads=H // 4, dim=hd, vdim=hd, scale=hd ** -0.5, softcap=20.0, bias_max=512, mask=dict(size=window, keep_first=4))
+    side = {"type": "parallel", "mixer": dict(left=left, left_scale=0.6, right=dict(heads=gheads, dim=gdim, vdim=gvdim, tau=16.0), right_scale=1.1), "mlp": dict(mlp, limit=7.0)}
+    return {"stack": {"architecture": "Tupitar", "vocab": V, "width": E, "max_positions": max_positions, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6}, "layers": [at, mb] * (L // 2)},
+            "mafurax": {"architecture": "Mafurax", "vocab": V, "width": E, "logit_scale": E ** -0.5, "norm": {"eps": 1e-6}, "layers": [side] * L}}
 
 
 def stack_bench():
-    """Random weights, one GPU, one process.  Per size: the stack (bfloat16) and a Llama Q4_K_M GGUF with the same width, feed-forward, heads, layer count and vocabulary:
+    """Random weights, one GPU, one process.  Per size: the stacks of both designs (bfloat16) and a Llama Q4_K_M GGUF with the same width, feed-forward, heads, layer count and vocabulary:
     a 2048-token prompt (and shorter ones), greedy decoding behind it, sixteen sequences decoded together (stack only: Llama contexts hold one), and one decode step with an
     event pair around every launch (us and GB/s of algorithmic bytes per launch kind; `of_hbm` = fraction of the 8 TB/s peak)."""
     import tempfile
@@ -596,7 +599,8 @@ def stack_bench():
     from booster_amd.synthetic import write_synthetic_stack
     bbuild.build()
     d = tempfile.mkdtemp(prefix="bamd_stack_", dir="/dev/shm" if os.path.isdir("/dev/shm") else None)
-    sizes = {"2048": dict(E=2048, F=8192, H=16, hd=128, R=256, mheads=64, P=64, state=128, L=8), "4096": dict(E=4096, F=14336, H=32, hd=128, R=512, mheads=128, P=64, state=128, L=8)}
+    sizes = {"2048": dict(E=2048, F=8192, H=16, hd=128, R=256, mheads=64, P=64, state=128, gheads=16, gdim=128, gvdim=128, window=1024, L=8),
+             "4096": dict(E=4096, F=14336, H=32, hd=128, R=512, mheads=128, P=64, state=128, gheads=32, gdim=128, gvdim=128, window=1024, L=8)}
     out = dict(metric="configured layer stack beside Llama Q4_K_M at equal layer sizes", data="synthetic", unit="tokens/s", n_gpus=1, sizes={})
 
     def run(m, V, E, n_seq, matrix_params):
@@ -641,18 +645,19 @@ def stack_bench():
         return r
     try:
         for name, z in sizes.items():
-            cfg = stack_config(**z)
-            E, F, L, V = z["E"], z["F"], z["L"], cfg["vocab"]
-            p = os.path.join(d, "stack"); write_synthetic_stack(p, cfg)
-            m = booster_amd.Model(p)
-            a = run(m, V, E, 16, m.weight_bytes / 2 - V * E)
-            m.close(); shutil.rmtree(p)
+            E, F, L, res = z["E"], z["F"], z["L"], {}
+            for kind, cfg in stack_configs(**z).items():
+                V = cfg["vocab"]
+                p = os.path.join(d, "stack"); write_synthetic_stack(p, cfg)
+                m = booster_amd.Model(p)
+                res[kind] = run(m, V, E, 16, m.weight_bytes / 2 - V * E)
+                m.close(); shutil.rmtree(p)
             p = os.path.join(d, "llama.gguf"); Hkv = z["H"] // 4
             gguf.write_synthetic_llama(p, E=E, H=z["H"], Hkv=Hkv, L=L, F=F, V=V, seed=7, reuse_layers=True)
             m = booster_amd.Model(p)
             b = run(m, V, E, 1, L * (2.0 * E * E + 2.0 * E * Hkv * z["hd"] + 3.0 * E * F))
             m.close(); os.remove(p)
-            out["sizes"][name] = dict(shape=z, stack=a, llama_q4_k_m=b)
+            out["sizes"][name] = dict(shape=z, **res, llama_q4_k_m=b)
     finally:
         shutil.rmtree(d, ignore_errors=True)
     return out

@@ -79,6 +79,10 @@ def lib():
         L.bamd_op_group_norm.argtypes = [ci, vp, vp, ci, cf, ci, ci, vp]
         L.bamd_op_ssm.argtypes = [vp, ci, ci, ci, ci, ci, ci, ci, vp, vp, vp, vp, vp, vp, vp, vp]
         L.bamd_op_latent_attention.argtypes = [ci, vp, vp, vp, ci, vp, ci, ci, ci, ci, ci, cf, cf, vp, vp, vp, vp, ci, vp]
+        L.bamd_op_layer_rows.argtypes = [ci, vp, vp, vp, vp, cf, ci, ci, vp, vp]
+        L.bamd_op_clamped_glu.argtypes = [ci, vp, vp, cf, ci, ci, vp]
+        L.bamd_op_kv_attention.argtypes = [ci, vp, vp, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, cf, cf, cf, ci, vp, ci, ci, ci, ci, cf, ci, vp]
+        L.bamd_op_gated_linear.argtypes = [ci, vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, ci, ci, ci, ci, cf, cf, cf, cf, ci, vp, vp, vp]
         L.bamd_set_aql.argtypes = [ci]; L.bamd_set_aql.restype = None
         L.bamd_aql_runs.argtypes = [vp]
         _lib = L
@@ -408,3 +412,39 @@ def op_latent_attention(q, c, gate, past, uk, uv, c_norm, sink, scale, eps, dtyp
     out = np.zeros((T, H, vdim), np.float32)
     _chk(lib().bamd_op_latent_attention(_act(dtype), _p(q), _p(c), _p(gate), T, _p(past), pos0, H, dim, vdim, c.shape[1], scale, eps, _p(c_norm), _p(uk), _p(uv), _p(sink), int(decode), _p(out)))
     return out
+
+
+def op_layer_rows(x, y, g, gi, eps, dtype):
+    """returns (x' = x + layer norm of y, layer norm of x'); y None: x' = x, gi None: no second norm"""
+    x, y, g, gi = map(_f32, (x, y, g, gi))
+    xo, h = np.zeros_like(x), np.zeros_like(x)
+    _chk(lib().bamd_op_layer_rows(_act(dtype), _p(x), _p(y), _p(g), _p(gi), eps, x.shape[0], x.shape[1], _p(xo), _p(h)))
+    return xo, h
+
+
+def op_clamped_glu(gate, up, limit, dtype):
+    gate, up = _f32(gate), _f32(up)
+    out = np.zeros_like(gate)
+    _chk(lib().bamd_op_clamped_glu(_act(dtype), _p(gate), _p(up), limit, gate.shape[0], gate.shape[1], _p(out)))
+    return out
+
+
+def op_kv_attention(q, k, v, gate, past_k, past_v, scale, cap, eps, unit, rel, bias_max, window, keep, dtype, out_scale=1.0, splits=0):
+    """q [T, H, dim], k [T, G, dim], v [T, G, vdim]; past_k / past_v: cached rows in front; rel [rows, H] bias table; splits > 0: the decoding kernel (T = 1).  Returns [T, H, vdim]"""
+    q, k, v, gate, past_k, past_v, rel = map(_f32, (q, k, v, gate, past_k, past_v, rel))
+    T, H, dim = q.shape
+    out = np.zeros((T, H, v.shape[2]), np.float32)
+    _chk(lib().bamd_op_kv_attention(_act(dtype), _p(q), _p(k), _p(v), _p(gate), T, _p(past_k), _p(past_v), 0 if past_k is None else len(past_k), H, k.shape[1], dim, v.shape[2], scale, cap, eps, int(unit),
+                                    _p(rel), 0 if rel is None else len(rel), bias_max, window, keep, out_scale, splits, _p(out)))
+    return out
+
+
+def op_gated_linear(q, k, v, gate, low, a2, a2b, norm, pos0, tau, q_scale, eps, state, dtype, out_scale=1.0, segment=0):
+    """q, k [T, H, dim], v, gate [T, H, vdim], low [T, rank], a2 [H * dim, rank] bit patterns, state [H, dim, vdim].  Returns (recurrence outputs, normed and gated, state)"""
+    q, k, v, gate, low, a2b, norm = map(_f32, (q, k, v, gate, low, a2b, norm))
+    a2, state = np.ascontiguousarray(a2, np.uint16), np.array(state, np.float32)
+    T, H, dim = q.shape
+    y, out = np.zeros_like(v), np.zeros_like(v)
+    _chk(lib().bamd_op_gated_linear(_act(dtype), _p(q), _p(k), _p(v), _p(gate), _p(low), _p(a2), _p(a2b), _p(norm), T, pos0, H, dim, v.shape[2], low.shape[1], tau, q_scale, eps, out_scale, segment,
+                                    _p(state), _p(y), _p(out)))
+    return y, out, state

@@ -1194,3 +1194,114 @@ BAMD_OP bamd_op_latent_attention(int act, const float * q, const float * c, cons
     for (int r = 0; r < rows; ++r) for (int h = 0; h < heads; ++h) memcpy(out + ((size_t) r * heads + h) * vdim, &wide[(size_t) r * HD + h * D], (size_t) vdim * 4);
     return 0;
 }
+BAMD_OP bamd_op_layer_rows(int act, const float * x, const float * y, const float * g, const float * gi, float eps, int rows, int E, float * xo, float * h) {
+    OpScratch s; bamd_batch_dev b; bamd_residual_args a; memset(&a, 0, sizeof a);
+    if (!x || !xo || !h || (y && !g) || rows < 1 || E < 1 || s.init(act) || s.one_entry(rows, 0, b)) return fail("bamd_op_layer_rows: bad arguments");
+    const size_t n = (size_t) rows * E;
+    float * dx, * dy = nullptr, * dg = nullptr, * di = nullptr, * dxo; void * dh;
+    if (s.up_(x, n, &dx) || (y && (s.up_(y, n, &dy) || s.up_(g, (size_t) E, &dg))) || (gi && s.up_(gi, (size_t) E, &di)) || s.alloc((void **) &dxo, n * 4) || s.alloc(&dh, (size_t) rows * up(E, 32) * 4)) return 1;
+    a.norm = BAMD_NORM_LAYER; a.x = dx; a.y = dy; a.ldy = E; a.g = dg; a.gi = di; a.eps = eps; a.xo = dxo; a.h = dh; a.E = E; a.ldh = up(E, 32);
+    bamd_launch_residual_rows(act, b, a, s.l.s);
+    HIPC(hipGetLastError());
+    return s.rows_back(dxo, rows, E, E, xo, true) || s.rows_back(dh, rows, E, a.ldh, h, act == BAMD_ACT_F32);
+}
+BAMD_OP bamd_op_clamped_glu(int act, const float * gate, const float * upv, float limit, int rows, int F, float * out) {
+    OpScratch s; float * dz; void * dh;
+    if (!gate || !upv || !out || rows < 1 || F < 1 || s.init(act)) return fail("bamd_op_clamped_glu: bad arguments");
+    const int ldh = up(F, 32);
+    std::vector<float> z((size_t) rows * 2 * ldh, 0.f);
+    for (int r = 0; r < rows; ++r) for (int i = 0; i < F; ++i) { float * p = &z[(size_t) r * 2 * ldh + (i / 16) * 32 + i % 16]; p[0] = gate[(size_t) r * F + i]; p[16] = upv[(size_t) r * F + i]; }
+    if (s.up_(z.data(), z.size(), &dz) || s.alloc(&dh, (size_t) rows * ldh * 4)) return 1;
+    bamd_launch_glu_rows(act, rows, { dz, 2 * ldh, limit, dh, ldh }, s.l.s);
+    HIPC(hipGetLastError());
+    return s.rows_back(dh, rows, F, ldh, out, act == BAMD_ACT_F32);
+}
+// past_k, past_v: what the cache holds in front of the rows (keys as they are cached), [pos0][kv_heads][dim / vdim]; rel: [rel_rows][heads] or null; splits: shares of a decoded row
+BAMD_OP bamd_op_kv_attention(int act, const float * q, const float * k, const float * v, const float * gate, int rows, const float * past_k, const float * past_v, int pos0, int heads, int kv_heads, int dim, int vdim,
+                             float scale, float cap, float eps, int unit, const float * rel, int rel_rows, int bias_max, int window, int keep, float out_scale, int splits, float * out) {
+    OpScratch s; bamd_batch_dev b; bamd_kv_args a; memset((void *) &a, 0, sizeof a);
+    if (!q || !k || !v || !out || rows < 1 || pos0 < 0 || (pos0 && (!past_k || !past_v)) || heads < 1 || kv_heads < 1 || heads % kv_heads || dim < 1 || dim > 256 || vdim < 1 || vdim > 256 || window < 1 || keep < 0 || splits > 64 ||
+        (splits && rows != 1) || (rel && (rel_rows < 2 || bias_max <= rel_rows / 2)) || s.init(act) || s.one_entry(rows, pos0, b)) return fail("bamd_op_kv_attention: bad arguments");
+    int D = 32; while (D < std::max(dim, vdim)) D *= 2;
+    const int H = heads, G = kv_heads, ld = up((H + 2 * G) * D + H, 16), kr = up(pos0 + rows, BAMD_PAGE), n_pg = kr / BAMD_PAGE, tq = bamd_kv_prompt_rows(act, D);
+    a.ld = ld; a.q_off = 0; a.k_off = H * D; a.v_off = (H + G) * D; a.g_off = (H + 2 * G) * D; a.heads = H; a.kv_heads = G; a.D = D; a.dim = dim; a.eps = eps; a.scale = scale; a.cap = cap; a.unit = unit; a.gated = gate ? 1 : 0;
+    a.window = window; a.keep = keep; a.out_scale = out_scale; a.ldo = H * D;
+    std::vector<float> in((size_t) rows * ld, 0.f), fk((size_t) kr * G * D, 0.f), fv((size_t) kr * G * D, 3.f);      // (whatever lies behind the past must not matter)
+    for (int r = 0; r < rows; ++r) {
+        float * p = &in[(size_t) r * ld];
+        for (int h = 0; h < H; ++h) { memcpy(p + h * D, q + ((size_t) r * H + h) * dim, (size_t) dim * 4); if (gate) p[a.g_off + h] = gate[(size_t) r * H + h]; }
+        for (int g = 0; g < G; ++g) { memcpy(p + a.k_off + g * D, k + ((size_t) r * G + g) * dim, (size_t) dim * 4); memcpy(p + a.v_off + g * D, v + ((size_t) r * G + g) * vdim, (size_t) vdim * 4); }
+    }
+    // page i of the sequence lies at place n_pg - 1 - i
+    for (int p = 0; p < pos0; ++p) for (int g = 0; g < G; ++g) {
+        const size_t at = ((size_t) (n_pg - 1 - p / BAMD_PAGE) * G + g) * BAMD_PAGE * D;
+        for (int i = 0; i < dim; ++i) fk[at + (size_t) (p % BAMD_PAGE) * D + i] = past_k[((size_t) p * G + g) * dim + i];
+        for (int i = 0; i < D; ++i) fv[at + (size_t) i * BAMD_PAGE + p % BAMD_PAGE] = i < vdim ? past_v[((size_t) p * G + g) * vdim + i] : 0.f;
+    }
+    float * din, * po, * pm, * db = nullptr; bamd_qtile * tiles; int32_t * kblk; void * o;
+    std::vector<bamd_qtile> t; for (int q0 = 0; q0 < rows; q0 += tq) t.push_back({ 0, q0 });
+    std::vector<int32_t> kb((size_t) n_pg, 0);
+    if (rel) { a.bias_top = bias_max; const std::vector<float> e = expand_bias(std::vector<float>(rel, rel + (size_t) rel_rows * H), rel_rows, H, bias_max); if (s.up_(e.data(), e.size(), &db)) return 1; }
+    const size_t cells = (size_t) bamd_kv_groups(a) * std::max(splits, 1);
+    if (s.up_(in.data(), in.size(), &din) || s.act_rows(fk.data(), kr, G * D, G * D, &a.kc) || s.act_rows(fv.data(), kr, G * D, G * D, &a.vc) || s.up_(t.data(), t.size(), &tiles) || s.up_(kb.data(), kb.size(), &kblk) ||
+        s.alloc(&o, (size_t) rows * H * D * 4) || s.alloc((void **) &po, cells * 16 * D * 4) || s.alloc((void **) &pm, cells * 128)) return 1;
+    a.in = din; a.bias = db; a.out = o;
+    int rc;
+    if (splits) rc = bamd_launch_kv_decode(act, b, a, po, pm, splits, s.l.s);
+    else { bamd_launch_kv_store(act, b, a, kblk, kr, s.l.s); rc = bamd_launch_kv_prompt(act, b, a, tiles, (int) t.size(), s.l.s); }
+    if (rc) return fail("bamd_op_kv_attention: unsupported shape");
+    HIPC(hipGetLastError());
+    std::vector<float> wide((size_t) rows * H * D);
+    if (s.rows_back(o, rows, H * D, H * D, wide.data(), act == BAMD_ACT_F32)) return 1;
+    for (int r = 0; r < rows; ++r) for (int h = 0; h < H; ++h) memcpy(out + ((size_t) r * H + h) * vdim, &wide[((size_t) r * H + h) * D], (size_t) vdim * 4);
+    return 0;
+}
+// q, k [rows][heads][dim], v, gate [rows][heads][vdim], low [rows][rank], a2 bfloat16 [heads * dim][rank]; state [heads][dim][vdim]; segment: tokens per scan segment (0: one).
+// y: outputs of the recurrence, out: normed and gated
+BAMD_OP bamd_op_gated_linear(int act, const float * q, const float * k, const float * v, const float * gate, const float * low, const uint16_t * a2, const float * a2b, const float * norm, int rows, int pos0, int heads, int dim,
+                             int vdim, int rank, float tau, float q_scale, float eps, float out_scale, int segment, float * state, float * y, float * out) {
+    OpScratch s; bamd_batch_dev b; bamd_gla_args a; memset((void *) &a, 0, sizeof a);
+    if (!q || !k || !v || !low || !a2 || !a2b || !norm || !state || !y || !out || rows < 1 || heads < 1 || dim < 1 || dim > 256 || vdim < 1 || rank < 1 || rank > 1024 || segment < 0 || s.init(act) || s.one_entry(rows, pos0, b))
+        return fail("bamd_op_gated_linear: bad arguments");
+    const int H = heads, Np = up(dim, 4), Pp = up(vdim, 4), ch = H * Np;
+    a.q_off = 0; a.k_off = ch; a.v_off = 2 * ch; a.g_off = a.v_off + H * Pp; a.t_off = a.g_off + H * Pp; a.ld = up(a.t_off + rank, 16); a.rank = rank; a.inv_tau = 1.f / tau; a.q_scale = q_scale; a.ldy = H * Pp;
+    a.heads = H; a.Np = Np; a.Pp = Pp; a.P = vdim; a.eps = eps; a.out_cols = up(H * Pp, 32); a.ldo = a.out_cols;
+    std::vector<float> in((size_t) rows * a.ld, 0.f), st((size_t) ch * Pp, 0.f), bias((size_t) ch, 0.f), nm((size_t) Pp, 0.f);
+    std::vector<uint16_t> w((size_t) rank * ch, 0);
+    for (int r = 0; r < rows; ++r) {
+        float * p = &in[(size_t) r * a.ld];
+        for (int h = 0; h < H; ++h) {
+            memcpy(p + h * Np, q + ((size_t) r * H + h) * dim, (size_t) dim * 4); memcpy(p + a.k_off + h * Np, k + ((size_t) r * H + h) * dim, (size_t) dim * 4); memcpy(p + a.v_off + h * Pp, v + ((size_t) r * H + h) * vdim, (size_t) vdim * 4);
+            if (gate) memcpy(p + a.g_off + h * Pp, gate + ((size_t) r * H + h) * vdim, (size_t) vdim * 4);
+        }
+        memcpy(p + a.t_off, low + (size_t) r * rank, (size_t) rank * 4);
+    }
+    if (!gate) a.g_off = -1;
+    for (int h = 0; h < H; ++h) for (int i = 0; i < dim; ++i) {
+        bias[(size_t) h * Np + i] = a2b[h * dim + i];
+        for (int r = 0; r < rank; ++r) w[(size_t) r * ch + h * Np + i] = a2[((size_t) h * dim + i) * rank + r];
+        memcpy(&st[((size_t) h * Np + i) * Pp], state + ((size_t) h * dim + i) * vdim, (size_t) vdim * 4);
+    }
+    for (int i = 0; i < vdim; ++i) nm[(size_t) i] = norm[i] * out_scale;
+    std::vector<bamd_segment> seg;
+    const int len = segment ? segment : rows;
+    for (int t = 0; t < rows; t += len) seg.push_back({ 0, t, std::min(len, rows - t), 0, 0 });
+    for (bamd_segment & g : seg) g.last = (int) seg.size() - 1;
+    float * din, * ds, * db, * dn, * dy; uint16_t * dw; bamd_segment * dseg; void * o;
+    if (s.up_(in.data(), in.size(), &din) || s.up_(st.data(), st.size(), &ds) || s.up_(bias.data(), bias.size(), &db) || s.up_(nm.data(), nm.size(), &dn) || s.up_(w.data(), w.size(), &dw) || s.up_(seg.data(), seg.size(), &dseg) ||
+        s.alloc((void **) &dy, (size_t) rows * H * Pp * 4) || s.alloc(&o, (size_t) rows * a.ldo * 4) || s.alloc((void **) &a.alpha, (size_t) rows * ch * 4) || s.alloc((void **) &a.seg_state, seg.size() * ch * Pp * 4) ||
+        s.alloc((void **) &a.seg_decay, seg.size() * ch * 4)) return 1;
+    a.in = din; a.a2 = dw; a.a2b = db; a.norm = dn; a.state = ds; a.y = dy; a.out = o;
+    if (bamd_launch_gla(b, a, rows, dseg, (int) seg.size(), s.l.s)) return fail("bamd_op_gated_linear: unsupported shape");
+    bamd_launch_gla_norm(act, a, rows, s.l.s);
+    HIPC(hipGetLastError());
+    std::vector<float> wy((size_t) rows * H * Pp), wo(wy.size());
+    if (s.rows_back(dy, rows, H * Pp, H * Pp, wy.data(), true) || s.rows_back(o, rows, H * Pp, a.ldo, wo.data(), act == BAMD_ACT_F32)) return 1;
+    HIPC(hipMemcpy(st.data(), ds, st.size() * 4, hipMemcpyDeviceToHost));
+    for (int r = 0; r < rows; ++r) for (int h = 0; h < H; ++h) {
+        memcpy(y + ((size_t) r * H + h) * vdim, &wy[((size_t) r * H + h) * Pp], (size_t) vdim * 4);
+        memcpy(out + ((size_t) r * H + h) * vdim, &wo[((size_t) r * H + h) * Pp], (size_t) vdim * 4);
+    }
+    for (int h = 0; h < H; ++h) for (int i = 0; i < dim; ++i) memcpy(state + ((size_t) h * dim + i) * vdim, &st[((size_t) h * Np + i) * Pp], (size_t) vdim * 4);
+    return 0;
+}

@@ -1,4 +1,4 @@
-"""GPU: the configured layer stacks (Tupitar) against oracle/stack_oracle.py — every mechanism alone, whole models in both compute types, and what must not matter:
+"""GPU: the configured layer stacks (Tupitar, Mafurax) against oracle/stack_oracle.py — every mechanism alone, whole models in both compute types, and what must not matter:
 portions, batches, pages and sequences."""
 import ctypes as C
 import json
@@ -11,7 +11,7 @@ import pytest
 
 from conftest import ROOT
 from oracle import stack_oracle as so
-from stack_cases import CONFIGS, SEEDS, config, latent, mamba, tokens
+from stack_cases import CONFIGS, ROWS, SEEDS, attend, config, latent, mafurax, mamba, parallel, tokens
 
 pytestmark = pytest.mark.gpu
 TOL = {"float32": 3e-5, "bfloat16": 0.03}                 # of the reference's root mean square
@@ -199,9 +199,9 @@ def test_sinks_and_gates(bamd, dtype, decode):
 
 # ---- whole models ------------------------------------------------------------------------------------------------------------------------------------------
 class Case:
-    def __init__(self, folder, cfg, seed):
+    def __init__(self, folder, cfg, seed, rows=None):
         self.folder, self.cfg = folder, cfg
-        w = so.random_model(cfg, seed)
+        w = so.random_model(cfg, seed, rows)
         so.write_model(folder, cfg, w)
         self.oracle = so.StackModel(cfg, w)
         self.known = {}
@@ -216,7 +216,7 @@ class Case:
 @pytest.fixture(scope="module")
 def cases(tmp_path_factory):
     d = tmp_path_factory.mktemp("stack")
-    return {n: Case(str(d / n), c, SEEDS[n]) for n, c in sorted(CONFIGS.items())}
+    return {n: Case(str(d / n), c, SEEDS[n], ROWS.get(n)) for n, c in sorted(CONFIGS.items())}
 
 
 @pytest.fixture(params=[(n, t) for n in sorted(CONFIGS) for t in DTYPES], ids=lambda p: "-".join(p))
@@ -357,9 +357,10 @@ def test_greedy_generation(run):
         assert [int(o[0]) for o in out] == first[:4] and [o[0] for o in sched] == first
 
 
-def test_long_decoding(bamd, cases):
+@pytest.mark.parametrize("name", ["odd", "side", "side_long"])
+def test_long_decoding(bamd, cases, name):
     """hundreds of decoded tokens behind a short prompt: in one device loop, then token by token, over page borders; the state of a sequence beside it stays"""
-    case = cases["odd"]
+    case = cases[name]
     m = bamd.Model(case.folder, dtype="float32"); c = bamd.Context(m, 704, 2)
     p = tokens(case.cfg, 6, 3)
     c.decode_batch([(1, tokens(case.cfg, 9, 4), [])])
@@ -377,10 +378,15 @@ def test_long_decoding(bamd, cases):
     c.close(); m.close()
 
 
+@pytest.mark.parametrize("design", ["Tupitar", "Mafurax"])
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_many_wanted_places_and_passes(bamd, dtype, tmp_path):
-    """more rows than one pass holds (2048), more wanted places than the logits buffer, a prompt cut between passes, a wide latent and larger matrices"""
+def test_many_wanted_places_and_passes(bamd, dtype, design, tmp_path):
+    """more rows than one pass holds (2048), more wanted places than the logits buffer, a prompt cut between passes, a wide latent and larger matrices; scans in segments, a window and kept
+    tokens far behind the queries"""
     cfg = config(128, 97, [latent(2, 16, 24, 40, 0.3, ff=64), mamba(2, 12, 10, 1, 1, 4, ff=48)], max_positions=1600)
+    if design == "Mafurax":
+        cfg = mafurax(128, 97, [parallel(attend(4, 2, 16, 24, 0.5, 10.0, 120, 200, 9), 0.8, (2, 20, 24, 16.0), 1.0, ff=64, limit=1.0),
+                                parallel(attend(2, 1, 24, 16, 0.4, 12.0, 800, 900, 0), 0.8, (3, 12, 16, 16.0), 1.0, ff=48, limit=1.0)])
     case = Case(str(tmp_path / "m"), cfg, 3)
     m = bamd.Model(case.folder, dtype=dtype); c = bamd.Context(m, 3200, 3)
     t = [tokens(cfg, n, n) for n in (900, 1500, 40)]
@@ -421,11 +427,12 @@ def test_limits(bamd, cases):
         bamd.Model(case.folder + "_b")
 
 
+@pytest.mark.parametrize("name", ["odd", "side"])
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_layer_split_stages(bamd, cases, dtype):
+def test_layer_split_stages(bamd, cases, dtype, name):
     """the layers over two stages with the hidden state handed over: prompt, portions and single tokens"""
     import torch
-    case = cases["odd"]
+    case = cases[name]
     t = tokens(case.cfg, 150, 1)
     E = case.cfg["width"]
     a = bamd.Model(case.folder, layer_first=0, layer_last=1, with_output=False, dtype=dtype)
@@ -453,9 +460,10 @@ def test_layer_split_stages(bamd, cases, dtype):
         x.close()
 
 
-def test_replays_with_other_work_between(bamd, cases):
+@pytest.mark.parametrize("name", ["wide", "side_wide"])
+def test_replays_with_other_work_between(bamd, cases, name):
     """the decoding graph, replayed with prompts, other sequences and eager work between its replays, gives what a fresh context gives"""
-    case = cases["wide"]
+    case = cases[name]
     t = tokens(case.cfg, 80, 6)
     m = bamd.Model(case.folder, dtype="float32"); c = bamd.Context(m, 512, 3)
     c.decode_batch([(0, t[:40], [])])
@@ -495,9 +503,10 @@ def test_bridge_serves_a_model_folder(bamd, tmp_path):
     assert L.status(b"stack-a") == L.status(b"stack-b")
 
 
-def test_trace_run(bamd, cases, tmp_path):
+@pytest.mark.parametrize("name", ["odd", "side"])
+def test_trace_run(bamd, cases, name, tmp_path):
     """bin/trace_run replays requests step by step and writes the wanted logits"""
-    case = cases["odd"]
+    case = cases[name]
     t = tokens(case.cfg, 150, 1)
     steps = [{"step": 0, "entries": [{"id": "x", "tokens": t[:70], "want": [69, 3]}, {"id": "y", "tokens": t[:5], "want": []}], "end": []},
              {"step": 1, "entries": [{"id": "y", "tokens": [t[5]], "want": [0]}, {"id": "x", "tokens": [t[70]], "want": [0]}], "end": ["y"]},
@@ -517,11 +526,12 @@ def test_trace_run(bamd, cases, tmp_path):
         assert not (out / "2.f32").exists()
 
 
-def test_command_line(bamd, cases, capsys):
+@pytest.mark.parametrize("name", ["odd", "side"])
+def test_command_line(bamd, cases, name, capsys):
     """python -m booster_amd: several requests of a folder together; a GGUF model through the same scheduler, one request after the other"""
     from booster_amd.__main__ import main
     from conftest import GOLDEN
-    case = cases["odd"]
+    case = cases[name]
     prompts = [tokens(case.cfg, n, n) for n in (5, 70, 33)]
     assert main(["--model", case.folder, "--dtype", "float32", "-n", "6"] + [x for p in prompts for x in ("--tokens", ",".join(map(str, p)))]) == 0
     got = [[int(t) for t in l.split(",")] for l in capsys.readouterr().out.split()]

@@ -7,7 +7,7 @@ import numpy as np
 import pytest
 
 from oracle import stack_oracle as so
-from stack_cases import CONFIGS, SEEDS, tokens
+from stack_cases import CONFIGS, tokens, weights
 
 
 def rel(a, b):
@@ -18,7 +18,7 @@ def rel(a, b):
 @pytest.mark.parametrize("name", sorted(CONFIGS))
 def test_portions_of_the_plain_statement(name):
     cfg = CONFIGS[name]
-    m = so.StackModel(cfg, so.random_model(cfg, 1))
+    m = so.StackModel(cfg, weights(name, 1))
     t = tokens(cfg, 21, 2)
     whole = m.forward(t)
     st = m.new_state()
@@ -35,18 +35,22 @@ class Rounded:
     def __matmul__(self, x):
         return self.w @ so.round_bf16(x).astype(np.float64)
 
+    def __getitem__(self, i):
+        return self.w[i]
+
 
 @pytest.mark.parametrize("name", sorted(CONFIGS))
 def test_rounding_alone_stays_small(name):
     """what bfloat16 operands cost in the test models: less than half of the tolerance the GPU tests allow, at every position"""
     cfg = CONFIGS[name]
-    m = so.StackModel(cfg, so.random_model(cfg, SEEDS[name]))
+    m = so.StackModel(cfg, weights(name))
     t = tokens(cfg, 150, 1)
     exact = m.forward(t)
     for ly, mix, mlp, _ in m.layers:
-        for part, keys in ((mix, ("in", "q", "dkv", "g", "o")), (mlp, ("up", "down"))):
+        for part, keys in ((mix, ("in", "q", "dkv", "g", "o", "left.q", "left.k", "left.v", "left.g", "left.o", "right.q", "right.k", "right.v", "right.g", "right.o", "right.a1")), (mlp, ("gate", "up", "down"))):
             part.update({k: Rounded(part[k]) for k in keys if k in part})
-    m.w["head"] = Rounded(m.w["head"])
+    head = "head" if "head" in m.w else "embed"
+    m.w[head] = Rounded(m.w[head])
     e = np.sqrt(((m.forward(t) - exact) ** 2).mean(-1) / (exact ** 2).mean(-1))
     assert 0.001 < e.max() < 0.015
 
@@ -63,20 +67,51 @@ FAULTS = {
 }
 
 
-@pytest.mark.parametrize("fault", sorted(FAULTS))
-def test_a_fault_shows_in_the_logits(fault, monkeypatch):
+SIDE_FAULTS = {
+    "window one longer": ("visible", lambda i, j, m: j <= i and (i - j <= m["size"] or j < m["keep_first"])),
+    "window one shorter": ("visible", lambda i, j, m: j <= i and (i - j < m["size"] - 1 or j == i or j < m["keep_first"])),
+    "first tokens not kept": ("visible", lambda i, j, m: j <= i and i - j < m["size"]),
+    "one first token too many": ("visible", lambda i, j, m: j <= i and (i - j < m["size"] or j <= m["keep_first"])),
+    "scores not capped": ("softcap", lambda s, cap: s),
+    "bias in front of the cap": ("biased_softmax", lambda s, bias: (lambda e: e / e.sum())(np.exp(6 * np.tanh((s + bias) / 6)))),
+    "no bias": ("biased_softmax", lambda s, bias: np.exp(s) / np.exp(s).sum()),
+    "distances one off": ("distance_bucket", lambda n, rows, top, f=so.distance_bucket: f(n + 1, rows, top)),
+    "no logarithmic steps": ("distance_bucket", lambda n, rows, top: min(n, rows - 1)),
+    "no tau": ("gla_decay", lambda z, tau: so.sigmoid(z)),
+    "one decay per head": ("gla_step", lambda S, al, k, v, q: ((lambda n: (n, n.T @ q))(al.mean() * S + np.outer(k, v)))),
+    "decay on the columns": ("gla_step", lambda S, al, k, v, q: ((lambda n: (n, n.T @ q))(np.resize(al, len(v))[None] * S + np.outer(k, v)))),
+    "own token not decayed in": ("gla_step", lambda S, al, k, v, q: (al[:, None] * S + np.outer(k, v), (al[:, None] * S).T @ q)),
+    "state not carried": ("gla_step", lambda S, al, k, v, q: (np.outer(k, v), np.outer(k, v).T @ q)),
+    "mean not taken off": ("layer_norm", lambda x, w, eps: so.rms(x, eps) * w),
+    "no one behind up": ("clamped_glu", lambda g, u, limit: (lambda a: a * so.sigmoid(1.702 * a) * np.clip(u, -limit, limit))(np.minimum(g, limit))),
+    "gate clamped below": ("clamped_glu", lambda g, u, limit: (lambda a: a * so.sigmoid(1.702 * a) * (np.clip(u, -limit, limit) + 1))(np.clip(g, -limit, limit))),
+    "up not clamped": ("clamped_glu", lambda g, u, limit: (lambda a: a * so.sigmoid(1.702 * a) * (u + 1))(np.minimum(g, limit))),
+}
+
+
+@pytest.mark.parametrize("name,fault", [("odd", f) for f in sorted(FAULTS)] + [("side", f) for f in sorted(SIDE_FAULTS)])
+def test_a_fault_shows_in_the_logits(name, fault, monkeypatch):
     """every mechanism matters in the test models: a fault planted in the plain statement moves the logits far beyond the tolerances of the GPU tests"""
-    cfg = CONFIGS["odd"]
-    w = so.random_model(cfg, 3)
-    t = tokens(cfg, 24, 4)
+    cfg = CONFIGS[name]
+    w = weights(name, 3)
+    t = tokens(cfg, 70 if name == "side" else 24, 4)
     good = so.StackModel(cfg, w).forward(t)
-    monkeypatch.setattr(so, *FAULTS[fault])
-    assert rel(so.StackModel(cfg, w).forward(t), good) > 0.1
+    monkeypatch.setattr(so, *(FAULTS if name == "odd" else SIDE_FAULTS)[fault])
+    assert rel(so.StackModel(cfg, w).forward(t), good) > (0.1 if name == "odd" else 0.02)
+
+
+def test_buckets():
+    """the distances of every row: exact ones, then steps that grow, the last row from its start to infinity"""
+    got = [so.distance_bucket(n, 8, 32) for n in range(40)]
+    assert got[:4] == [0, 1, 2, 3] and got[4:7] == [4, 4, 4] and got[31:] == [7] * 9 and got == sorted(got)
+    assert [so.distance_bucket(n, 2, 9) for n in range(4)] == [0, 1, 1, 1]
+    m = {"size": 3, "keep_first": 2}
+    assert [[j for j in range(9) if so.visible(i, j, m)] for i in (0, 2, 4, 5, 8)] == [[0], [0, 1, 2], [0, 1, 2, 3, 4], [0, 1, 3, 4, 5], [0, 1, 6, 7, 8]]
 
 
 def test_weights_survive_the_file(tmp_path):
     cfg = CONFIGS["ones"]
-    w = so.random_model(cfg, 5)
+    w = weights("ones", 5)
     so.write_model(str(tmp_path / "m"), cfg, w)
     m = so.StackModel.load(str(tmp_path / "m"))
     assert m.cfg == cfg and set(m.w) == set(w) and all(np.array_equal(m.w[k], np.asarray(w[k], np.float64)) for k in w)
@@ -95,7 +130,7 @@ def test_registry_and_configuration_errors(tmp_path):
     w = so.random_model(cfg, 6)
     d = tmp_path / "m"
     so.write_model(str(d), dict(cfg, architecture="Nope"), w)
-    assert "Tupitar" in load_error(d) and "Nope" in load_error(d)
+    assert all(n in load_error(d) for n in ("Tupitar", "Mafurax", "Nope"))
     so.write_model(str(d), {k: v for k, v in cfg.items() if k != "width"}, w)
     assert "width" in load_error(d)
     so.write_model(str(d), dict(cfg, layers=[]), w)
