@@ -13,7 +13,7 @@ LIB = os.path.join(HERE, "lib", "libbooster_amd.so")
 # the kernels of a decode step are ALSO built as raw gfx950 code objects (same sources, same flags) and embedded in the library: bamd_aql.cpp loads them through
 # HSA and replays a step from the library's own AQL queue (csrc/bamd_aql.h)
 DECODE_KERNEL_SOURCES = ["bamd_matvec.hip", "bamd_matvec_fast_a.hip", "bamd_matvec_fast_b.hip", "bamd_attention.hip", "bamd_colaunch.hip"]
-SOURCES = ["bamd_aql.cpp", "bamd_matvec.hip", "bamd_matvec_fast_a.hip", "bamd_matvec_fast_b.hip", "bamd_attention.hip", "bamd_attention_mfma.hip", "bamd_colaunch.hip", "bamd_prefill.hip", "bamd_prefill2.hip", "bamd_sampler.hip", "bamd_dense.hip", "bamd_rows.hip", "bamd_ssm.hip", "bamd_latent.hip", "bamd_kv.hip", "bamd_gla.hip", "bamd_arch.cpp", "bamd_stack.cpp", "bamd_engine.cpp", "bamd_gguf.cpp", "bamd_vocab.cpp", "bamd_bridge.cpp"]
+SOURCES = ["bamd_aql.cpp", "bamd_matvec.hip", "bamd_matvec_fast_a.hip", "bamd_matvec_fast_b.hip", "bamd_attention.hip", "bamd_attention_mfma.hip", "bamd_colaunch.hip", "bamd_prefill.hip", "bamd_prefill2.hip", "bamd_sampler.hip", "bamd_dense.hip", "bamd_rows.hip", "bamd_ssm.hip", "bamd_latent.hip", "bamd_kv.hip", "bamd_gla.hip", "bamd_pair.hip", "bamd_arch.cpp", "bamd_stack.cpp", "bamd_engine.cpp", "bamd_gguf.cpp", "bamd_vocab.cpp", "bamd_bridge.cpp"]
 HEADERS = ["bamd_runtime.h", "bamd_arch.h", "bamd_stack.h", "bamd_dense.h", "bamd_dense_device.h", "bamd_kv_device.h", "bamd_gla_device.h", "bamd_json.h", "bamd_safetensors.h", "bamd_aql.h", "bamd_formats.h", "bamd_kernels.h", "bamd_device.h", "bamd_matvec_core.h", "bamd_attn_fused.h", "bamd_mfma_common.h", "bamd_gguf.h", "bamd_vocab.h", "bamd_unicode_tables.h", "../../include/bamd.h", "../../include/booster_bridge.h"]
 # -ffp-contract=off: the numerics contract (bit-parity with the reference CPU path) forbids implicit FMA fusion.
 # -fno-slp-vectorize (decode kernels only, NO_SLP): SLP packs neighbouring f32 multiplies into v_pk_mul_f32, whose operands need
@@ -25,7 +25,7 @@ NO_SLP = ("bamd_matvec.hip", "bamd_matvec_fast_a.hip", "bamd_matvec_fast_b.hip",
 KERNARG_PRELOAD = {"bamd_matvec_fast_a.hip": ["-mllvm", "-amdgpu-kernarg-preload-count=16"], "bamd_matvec_fast_b.hip": ["-mllvm", "-amdgpu-kernarg-preload-count=16"]}
 # -packed-fp32-ops: no v_pk_{add,mul,fma}_f32 anywhere (some of their forms have given wrong results on this hardware); the host pass only warns about the name.
 # the layer stacks carry no bit-parity contract: products and sums may fuse
-CONTRACT = ("bamd_dense.hip", "bamd_rows.hip", "bamd_ssm.hip", "bamd_latent.hip", "bamd_kv.hip", "bamd_gla.hip")
+CONTRACT = ("bamd_dense.hip", "bamd_rows.hip", "bamd_ssm.hip", "bamd_latent.hip", "bamd_kv.hip", "bamd_gla.hip", "bamd_pair.hip")
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-ffp-contract=off", "-fPIC", "-fvisibility=hidden", "-Wno-unused-result", "-Wno-unused-value"]
 
 

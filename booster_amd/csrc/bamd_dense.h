@@ -126,6 +126,7 @@ int bamd_kv_span(const bamd_kv_args & a, int pages);
 // decoding: one row per entry, its own key and value stored as well.  part_o [rows][kv_heads x head groups][splits][16][D], part_ml [..][16][2]
 int bamd_launch_kv_decode(int act, const bamd_batch_dev & b, const bamd_kv_args & a, float * part_o, float * part_ml, int splits, hipStream_t s);
 int bamd_kv_groups(const bamd_kv_args & a);        // kv_heads x ceil(heads per kv head / 16)
+bool bamd_kv_valid(const bamd_kv_args & a);
 
 // ---- gated linear attention -------------------------------------------------------------------------------------------------------------------------
 // S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t with alpha = sigmoid(a2 t + b)^(1 / tau) per key channel
@@ -148,3 +149,8 @@ struct bamd_segment { int32_t entry, t0, n, first, last; };       // first, last
 int bamd_launch_gla(const bamd_batch_dev & b, const bamd_gla_args & a, int max_n, const bamd_segment * segs, int n_segs, hipStream_t s);
 void bamd_launch_gla_norm(int act, const bamd_gla_args & a, int rows, hipStream_t s);
 int bamd_gla_blocks(int heads, int Pp);            // blocks of one segment
+bool bamd_gla_valid(const bamd_gla_args & a);
+
+// ---- both at once ------------------------------------------------------------------------------------------------------------------------------------
+// a decoded token through attention and gated linear attention that read the same projection: their blocks share two launches
+int bamd_launch_kv_gla_decode(int act, const bamd_batch_dev & b, const bamd_kv_args & kv, const bamd_gla_args & gla, float * part_o, float * part_ml, int splits, hipStream_t s);

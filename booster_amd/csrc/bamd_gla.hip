@@ -64,13 +64,10 @@ __global__ void __launch_bounds__(256) gla_join_kernel(bamd_batch_dev b, bamd_gl
         s = next;
     }
 }
-// block (four heads, row)
-template <typename T> __global__ void __launch_bounds__(256) gla_norm_kernel(bamd_gla_args a) {
-    const int h = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (h < a.heads) gla_norm_wave<T>(a, h, blockIdx.y);
-}
+// block (sixteen heads, row)
+template <typename T> __global__ void __launch_bounds__(256) gla_norm_kernel(bamd_gla_args a) { gla_norm_block<T>(a, blockIdx.x * 16, blockIdx.y); }
 void bamd_launch_gla_norm(int act, const bamd_gla_args & a, int rows, hipStream_t s) {
-    const dim3 grid((a.heads + 3) / 4, rows);
+    const dim3 grid((a.heads + 15) / 16, rows);
     if (act == BAMD_ACT_F32) hipLaunchKernelGGL(gla_norm_kernel<float>, grid, dim3(256), 0, s, a);
     else hipLaunchKernelGGL(gla_norm_kernel<bamd_bf>, grid, dim3(256), 0, s, a);
 }
@@ -94,10 +91,13 @@ template <int MODE> static int scan_pick(int pt, const bamd_batch_dev & b, const
     return pt == 16 ? scan_go<16, MODE>(b, a, segs, n_segs, many, s) : pt == 32 ? scan_go<32, MODE>(b, a, segs, n_segs, many, s) : scan_go<64, MODE>(b, a, segs, n_segs, many, s);
 }
 int bamd_gla_blocks(int heads, int Pp) { return (Pp + 63) / 64 * heads; }
+bool bamd_gla_valid(const bamd_gla_args & a) {
+    return a.Np >= 4 && a.Np <= 256 && !(a.Np & 3) && a.Pp >= 4 && !(a.Pp & 3) && a.heads >= 1 && a.rank >= 1 && a.rank <= 1024 && !((a.ld | a.q_off | a.k_off | a.v_off) & 3) && (a.g_off < 0 || !(a.g_off & 3)) && !((a.ldo | a.out_off) & 3);
+}
 int bamd_launch_gla(const bamd_batch_dev & b, const bamd_gla_args & a, int max_n, const bamd_segment * segs, int n_segs, hipStream_t s) {
-    if (a.Np < 4 || a.Np > 256 || (a.Np & 3) || a.Pp < 4 || (a.Pp & 3) || a.heads < 1 || a.rank < 1 || a.rank > 1024 || max_n < 1 || ((a.ld | a.q_off | a.k_off | a.v_off) & 3)) return 1;
+    if (!bamd_gla_valid(a) || max_n < 1) return 1;
     // enough blocks for the chip; narrower blocks only as far as they are filled
-    const long wide = (long) bamd_gla_blocks(a.heads, a.Pp) * n_segs;
+    const long wide = (long) bamd_gla_blocks(a.heads, a.Pp) * (max_n == 1 ? b.n_entries : n_segs);
     const int pt = a.Pp <= 16 || (max_n == 1 && wide * 2 < 256) ? 16 : a.Pp <= 32 || wide < 256 ? 32 : 64;
     if (max_n == 1) return scan_pick<GLA_STEP>(pt, b, a, nullptr, b.n_entries, false, s);
     if (!a.alpha) return 1;

@@ -7,7 +7,11 @@
 #include "bamd_dense_device.h"
 
 enum { GLA_STEP = 0, GLA_SCAN = 1, GLA_STATE = 2 };                // one decoded token (alpha computed here) | outputs and final state | final state and product of the decays only
-__device__ __forceinline__ float gla_alpha(float z, float inv_tau) { return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau); }     // sigmoid(z)^(1 / tau)
+// sigmoid(z)^(1 / tau): log2 of the sigmoid is min(z, 0) log2(e) - log2(1 + exp(-|z|)), right to an ulp of 1 + exp(-|z|), which is an ulp of the result
+__device__ __forceinline__ float gla_alpha(float z, float inv_tau) {
+    const float l = 1.4426950408889634f;
+    return __builtin_amdgcn_exp2f((fminf(z, 0.f) * l - __builtin_amdgcn_logf(1.f + __builtin_amdgcn_exp2f(-fabsf(z) * l))) * inv_tau);
+}
 
 template <int PT, int NPL, int MODE> struct GlaShape {
     static constexpr int Q = PT / 4, NG = 64 / Q, GROUPS = 4 * NG, NP = GROUPS * NPL, CT = MODE == GLA_STEP ? 1 : 8;      // NP >= Np state rows
@@ -71,7 +75,13 @@ __device__ __forceinline__ void gla_scan_block(const bamd_gla_args & a, int h, i
             for (int c = tid; c < Np; c += 256) {
                 ks[c] = in[a.k_off + h * Np + c]; qs[c] = in[a.q_off + h * Np + c];
                 float z = a.a2b[h * Np + c];
-                for (int r = 0; r < a.rank; ++r) z = fmaf(bf_f(a.a2[(size_t) r * aw + h * Np + c]), in[a.t_off + r], z);
+                for (int r0 = 0; r0 < a.rank; r0 += 16) {          // sixteen factors on their way at once
+                    float w[16], t[16];
+#pragma unroll
+                    for (int r = 0; r < 16; ++r) { const int i = min(r0 + r, a.rank - 1); w[r] = bf_f(a.a2[(size_t) i * aw + h * Np + c]); t[r] = in[a.t_off + i]; }
+#pragma unroll
+                    for (int r = 0; r < 16; ++r) z = fmaf(r0 + r < a.rank ? w[r] : 0.f, t[r], z);
+                }
                 as[c] = gla_alpha(z, a.inv_tau);
             }
         }
@@ -118,14 +128,35 @@ __device__ __forceinline__ void gla_scan_block(const bamd_gla_args & a, int h, i
         if constexpr (MODE == GLA_STATE) if (p0 == 0 && quad == 0) prod[r] = dec[j];
     }
 }
-// head h of a row: norm over its columns, gate; one wave
-template <typename T> __device__ __forceinline__ void gla_norm_wave(const bamd_gla_args & a, int h, int row) {
-    const int lane = threadIdx.x & 63;
-    const float * y = a.y + (size_t) row * a.ldy + h * a.Pp, * g = a.g_off >= 0 ? a.in + (size_t) row * a.ld + a.g_off + h * a.Pp : nullptr;
+// sixteen heads of a row from h0 on, sixteen lanes each: norm over a head's columns, gate; a whole block of 256
+template <typename T> __device__ __forceinline__ void gla_norm_block(const bamd_gla_args & a, int h0, int row) {
+    constexpr int RC = 4;
+    const int h = h0 + (threadIdx.x >> 4), l = (threadIdx.x & 15) * 4;
     T * out = (T *) a.out + (size_t) row * a.ldo + a.out_off;
-    float ss = 0.f;
-    for (int c = lane; c < a.Pp; c += 64) ss += y[c] * y[c];
-    const float r = 1.0f / sqrtf(wave_sum(ss) / (float) a.P + a.eps);
-    for (int c = lane; c < a.Pp; c += 64) out[h * a.Pp + c] = to_act<T>(y[c] * r * a.norm[c] * (g ? silu_f(g[c]) : 1.f));
-    if (h == a.heads - 1) for (int c = a.heads * a.Pp + lane; c < a.out_cols; c += 64) out[c] = to_act<T>(0.f);
+    if (h < a.heads) {
+        const float * y = a.y + (size_t) row * a.ldy + h * a.Pp, * g = a.g_off >= 0 ? a.in + (size_t) row * a.ld + a.g_off + h * a.Pp : nullptr;
+        bamd_v4 v[RC], gv[RC];
+        float ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < RC; ++c) {
+            const int i = l + c * 64;
+            v[c] = i < a.Pp ? *(const bamd_v4 *) (y + i) : bamd_v4{ 0, 0, 0, 0 };
+            if (g) gv[c] = i < a.Pp ? *(const bamd_v4 *) (g + i) : bamd_v4{ 0, 0, 0, 0 };
+#pragma unroll
+            for (int k = 0; k < 4; ++k) ss += v[c][k] * v[c][k];
+        }
+        for (int i = l + RC * 64; i < a.Pp; i += 64) { const bamd_v4 t = *(const bamd_v4 *) (y + i); for (int k = 0; k < 4; ++k) ss += t[k] * t[k]; }
+        const float r = 1.0f / sqrtf(row_sum16(ss) / (float) a.P + a.eps);
+        auto put = [&](int i, bamd_v4 t, bamd_v4 gate) {
+            t = t * r * *(const bamd_v4 *) (a.norm + i);
+            if (g)
+#pragma unroll
+                for (int k = 0; k < 4; ++k) t[k] *= gate[k] / (1.0f + __expf(-gate[k]));
+            store4<T>(out + h * a.Pp + i, t);
+        };
+#pragma unroll
+        for (int c = 0; c < RC; ++c) if (l + c * 64 < a.Pp) put(l + c * 64, v[c], gv[c]);
+        for (int i = l + RC * 64; i < a.Pp; i += 64) put(i, *(const bamd_v4 *) (y + i), g ? *(const bamd_v4 *) (g + i) : bamd_v4{ 0, 0, 0, 0 });
+    }
+    if (h0 + 16 >= a.heads) for (int c = a.heads * a.Pp + threadIdx.x; c < a.out_cols; c += 256) out[c] = to_act<T>(0.f);
 }

@@ -18,19 +18,49 @@ template <typename T> __global__ void __launch_bounds__(256) kv_store_kernel(bam
     const int lo = max(p0, e.pos0) - p0, hi = min(p0 + BAMD_PAGE, e.pos0 + e.n) - p0;      // places of the page that this step brings
     if (lo >= hi) return;
     const size_t at = ((size_t) b.pages[(size_t) e.seq * b.max_pages + pg] * a.kv_heads + g) * BAMD_PAGE * D;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    for (int c = lo + wave; c < hi; c += 4) {
-        const float * in = a.in + (size_t) (e.row0 + p0 + c - e.pos0) * a.ld, * k = in + a.k_off + g * D, * v = in + a.v_off + g * D;
-        float ss = 0.f;
-        for (int d = lane; d < D; d += 64) ss += k[d] * k[d];
-        ss = wave_sum(ss);
-        const float r = a.unit ? 1.0f / sqrtf(ss / (float) a.dim + a.eps) : 1.0f;
-        for (int d = lane; d < D; d += 64) { ((T *) a.kc)[at + (size_t) c * D + d] = to_act<T>(k[d] * r); vs[c * S + d] = to_act<T>(v[d]); }
+    // sixteen lanes per row, RU rows of a lane on their way at once
+    constexpr int RU = 2;
+    const int l = (threadIdx.x & 15) * 4, nc = (D + 63) / 64;
+    for (int c0 = lo + (threadIdx.x >> 4); c0 < hi; c0 += 16 * RU) {
+        bamd_v4 kv[RU][4], vv[RU][4];
+#pragma unroll
+        for (int u = 0; u < RU; ++u) {
+            const int c = min(c0 + 16 * u, hi - 1);
+            const float * in = a.in + (size_t) (e.row0 + p0 + c - e.pos0) * a.ld, * k = in + a.k_off + g * D, * v = in + a.v_off + g * D;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const bool live = i < nc && l + i * 64 < D;
+                kv[u][i] = live ? *(const bamd_v4 *) (k + l + i * 64) : bamd_v4{ 0, 0, 0, 0 }; vv[u][i] = live ? *(const bamd_v4 *) (v + l + i * 64) : bamd_v4{ 0, 0, 0, 0 };
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < RU; ++u) {
+            const int c = c0 + 16 * u;
+            float ss = 0.f;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) ss += kv[u][i][j] * kv[u][i][j];
+            ss = row_sum16(ss);
+            if (c >= hi) continue;
+            const float r = a.unit ? 1.0f / sqrtf(ss / (float) a.dim + a.eps) : 1.0f;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                if (i >= nc || l + i * 64 >= D) continue;
+                store4<T>((T *) a.kc + at + (size_t) c * D + l + i * 64, kv[u][i] * r);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) vs[c * S + l + i * 64 + j] = to_act<T>(vv[u][i][j]);
+            }
+        }
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < D * BAMD_PAGE; i += 256) {
+    for (int i = threadIdx.x * 4; i < D * BAMD_PAGE; i += 1024) {
         const int d = i / BAMD_PAGE, c = i % BAMD_PAGE;
-        if (c >= lo) ((T *) a.vc)[at + i] = c < hi ? vs[c * S + d] : to_act<T>(0.f);
+        bamd_v4 t;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) t[j] = c + j >= lo && c + j < hi ? (float) vs[(c + j) * S + d] : 0.f;
+        if (c >= lo) store4<T>((T *) a.vc + at + i, t);
+        else for (int j = 0; j < 4; ++j) if (c + j >= lo) ((T *) a.vc)[at + i + j] = to_act<T>(t[j]);
     }
 }
 
@@ -199,11 +229,11 @@ static int prompt_go(const bamd_batch_dev & b, const bamd_kv_args & a, const bam
     hipLaunchKernelGGL((kv_prompt_kernel<T, ND, RT>), dim3(n * a.heads), dim3(256), lds, s, b, a, tiles);
     return 0;
 }
-static bool valid(const bamd_kv_args & a) {
+bool bamd_kv_valid(const bamd_kv_args & a) {
     return a.heads >= 1 && a.kv_heads >= 1 && a.heads % a.kv_heads == 0 && a.window >= 1 && a.keep >= 0 && (!a.bias || a.bias_top >= 0) && !(a.ld & 3) && !(a.q_off & 3) && !(a.k_off & 3) && !(a.v_off & 3);
 }
 int bamd_launch_kv_prompt(int act, const bamd_batch_dev & b, const bamd_kv_args & a, const bamd_qtile * tiles, int n, hipStream_t s) {
-    if (n < 1 || !valid(a)) return 1;
+    if (n < 1 || !bamd_kv_valid(a)) return 1;
     if (act == BAMD_ACT_F32) switch (a.D) {
         case 32: return prompt_go<float, 1, 1>(b, a, tiles, n, s);
         case 64: return prompt_go<float, 2, 1>(b, a, tiles, n, s);
@@ -230,7 +260,7 @@ static int decode_go(const bamd_batch_dev & b, const bamd_kv_args & a, float * p
     return 0;
 }
 int bamd_launch_kv_decode(int act, const bamd_batch_dev & b, const bamd_kv_args & a, float * po, float * pm, int splits, hipStream_t s) {
-    if (splits < 1 || splits > 64 || !valid(a)) return 1;
+    if (splits < 1 || splits > 64 || !bamd_kv_valid(a)) return 1;
     if (act == BAMD_ACT_F32) switch (a.D) {
         case 32: return decode_go<float, 1>(b, a, po, pm, splits, s);
         case 64: return decode_go<float, 2>(b, a, po, pm, splits, s);

@@ -36,23 +36,31 @@ template <typename T> struct KvRow8 {
     }
 };
 // a head's row as operand pieces (lane / 16 takes columns lq * 8 .. + 8 of every 32), divided by its root mean square
-template <typename T, int ND> __device__ __forceinline__ void kv_head(const bamd_kv_args & a, const float * src, int lq, Frag<T> (&f)[ND]) {
-    KvRow8<T> r[ND];
+template <typename T, int ND> __device__ __forceinline__ void kv_head_load(const float * src, int lq, KvRow8<T> (&r)[ND]) {
+#pragma unroll
+    for (int k = 0; k < ND; ++k) r[k].load(src + k * 32 + lq * 8);
+}
+template <typename T, int ND> __device__ __forceinline__ void kv_head_norm(const bamd_kv_args & a, const KvRow8<T> (&r)[ND], Frag<T> (&f)[ND]) {
     float ss = 0.f;
 #pragma unroll
-    for (int k = 0; k < ND; ++k) { r[k].load(src + k * 32 + lq * 8); ss += r[k].squares(); }
+    for (int k = 0; k < ND; ++k) ss += r[k].squares();
     ss += __shfl_xor(ss, 16); ss += __shfl_xor(ss, 32);
     const float n = a.unit ? 1.0f / sqrtf(ss / (float) a.dim + a.eps) : 1.0f;
 #pragma unroll
     for (int k = 0; k < ND; ++k) r[k].put(f[k], n);
 }
+template <typename T, int ND> __device__ __forceinline__ void kv_head(const bamd_kv_args & a, const float * src, int lq, Frag<T> (&f)[ND]) {
+    KvRow8<T> r[ND];
+    kv_head_load<T, ND>(src, lq, r);
+    kv_head_norm<T, ND>(a, r, f);
+}
 
 // LDS of a decoding block: the waves' weights, then their sums
 template <typename T, int ND> struct KvDecodeLds {
-    static constexpr int D = ND * 32, NP = sizeof(T) == 2 ? 2 : 1, PS = 64 + 16 / sizeof(T);
+    static constexpr int D = ND * 32, NP = sizeof(T) == 2 ? 2 : 1, PS = 32 + 16 / sizeof(T);
     static constexpr size_t weights = (size_t) 4 * NP * 16 * PS * sizeof(T), sums = ((size_t) 4 * 16 * D + 4 * 16 * 2) * 4, bytes = weights > sums ? weights : sums;
 };
-// one of `splits` shares of a row's keys for (kv head, group of 16 heads) = y; four waves take pages in turn; the last wave of the last share brings the row's own key and value
+// one of `splits` shares of a row's keys for (kv head, group of 16 heads) = y; four waves take half pages in turn; the last wave of the last share brings the row's own key and value
 // and stores them in the cache
 template <typename T, int ND>
 __device__ __forceinline__ void kv_decode_block(const bamd_batch_dev & b, const bamd_kv_args & a, int sp, int splits, int y, int row, float * part_o, float * part_ml, unsigned char * lds) {
@@ -63,28 +71,60 @@ __device__ __forceinline__ void kv_decode_block(const bamd_batch_dev & b, const 
     const bamd_entry e = b.ent[row];
     const int pos = e.pos0, wi = sp * 4 + wave, nw = splits * 4;
     const KvPages pg(a, pos - a.window + 1, (pos + BAMD_PAGE - 1) / BAMD_PAGE);
-    const int per = (pg.count + nw - 1) / nw, t0 = wi * per, t1 = min(pg.count, t0 + per);
+    const int per = (2 * pg.count + nw - 1) / nw, t0 = wi * per, t1 = min(2 * pg.count, t0 + per);
     const bool own = wi == nw - 1;
     const int32_t * pages = b.pages + (size_t) e.seq * b.max_pages;
     const float * in = a.in + (size_t) row * a.ld;
     const KvCap cap = kv_cap(a);
     T * P = (T *) lds + (size_t) wave * NP * 16 * PS;
+    // everything the first 32 keys need is on its way before the queries are normed (heads too wide for the registers read them as they go)
+    constexpr bool AHEAD = ND * sizeof(T) <= 8;
+    Frag<T> kf[AHEAD ? 2 : 1][ND], vf[NV];
+    float bias[2][4];
+    const T * K = nullptr, * V = nullptr;
+    int k0 = 0;
+    auto request = [&](int i) {
+        const int p = pg.page(i >> 1), half = (i & 1) * 32;
+        const size_t at = ((size_t) pages[p] * a.kv_heads + g) * BAMD_PAGE * D;
+        K = (const T *) a.kc + at + (size_t) half * D; V = (const T *) a.vc + at + half; k0 = p * BAMD_PAGE + half;
+        if constexpr (AHEAD) {
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int k = 0; k < ND; ++k) kf[t][k].load(K + (t * 16 + lr) * D + k * 32 + lq * 8);
+#pragma unroll
+            for (int j = 0; j < NV; ++j) vf[j].load(V + (j * 16 + lr) * BAMD_PAGE + lq * 8);
+        }
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) bias[t][r] = kv_bias(a, h0 + min(lq * 4 + r, nh - 1), max(pos - (k0 + t * 16 + lr), 0));
+    };
+    KvRow8<T> qr[ND], kr[ND];
+    float vr[NV];
+    kv_head_load<T, ND>(in + a.q_off + (h0 + min(lr, nh - 1)) * D, lq, qr);
+    if (t0 < t1) request(t0);
+    if (own) {
+        kv_head_load<T, ND>(in + a.k_off + g * D, lq, kr);         // the same in every column
+#pragma unroll
+        for (int j = 0; j < NV; ++j) vr[j] = in[a.v_off + g * D + j * 16 + lr];
+    }
     Frag<T> q[ND];
-    kv_head<T, ND>(a, in + a.q_off + (h0 + min(lr, nh - 1)) * D, lq, q);
+    kv_head_norm<T, ND>(a, qr, q);
     bamd_v4 o[NV]; float m[4], l[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) { m[r] = -INFINITY; l[r] = 0.f; }
 #pragma unroll
     for (int j = 0; j < NV; ++j) o[j] = bamd_v4{ 0, 0, 0, 0 };
     // scores -> weights in LDS, running maximum and sum
-    auto weigh = [&](bamd_v4 (&sc)[4]) {
+    auto weigh = [&](bamd_v4 (&sc)[2]) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const float mx = fmaxf(m[r], row_max16(fmaxf(fmaxf(sc[0][r], sc[1][r]), fmaxf(sc[2][r], sc[3][r]))));
+            const float mx = fmaxf(m[r], row_max16(fmaxf(sc[0][r], sc[1][r])));
             const float al = mx == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m[r] - mx), ref = mx == -INFINITY ? 0.f : mx;
             float sum = 0.f;
 #pragma unroll
-            for (int t = 0; t < 4; ++t) {
+            for (int t = 0; t < 2; ++t) {
                 const float pe = __builtin_amdgcn_exp2f(sc[t][r] - ref);
                 sum += pe;
                 T * d = P + (lq * 4 + r) * PS + t * 16 + lr;
@@ -99,78 +139,74 @@ __device__ __forceinline__ void kv_decode_block(const bamd_batch_dev & b, const 
         wave_lds_fence();
     };
     for (int i = t0; i < t1; ++i) {
-        const int p = pg.page(i), k0 = p * BAMD_PAGE;
-        const size_t at = ((size_t) pages[p] * a.kv_heads + g) * BAMD_PAGE * D;
-        const T * K = (const T *) a.kc + at, * V = (const T *) a.vc + at;
-        bamd_v4 sc[4];
-        float bias[4][4];
+        bamd_v4 sc[2];
 #pragma unroll
-        for (int t = 0; t < 4; ++t)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) bias[t][r] = kv_bias(a, h0 + min(lq * 4 + r, nh - 1), max(pos - (k0 + t * 16 + lr), 0));
-#pragma unroll
-        for (int t = 0; t < 4; ++t) {
+        for (int t = 0; t < 2; ++t) {
             sc[t] = bamd_v4{ 0, 0, 0, 0 };
 #pragma unroll
-            for (int k = 0; k < ND; ++k) { Frag<T> kf; kf.load(K + (t * 16 + lr) * D + k * 32 + lq * 8); sc[t] = mma(q[k], kf, sc[t]); }
+            for (int k = 0; k < ND; ++k) {
+                if constexpr (!AHEAD) kf[0][k].load(K + (t * 16 + lr) * D + k * 32 + lq * 8);
+                sc[t] = mma(q[k], kf[AHEAD ? t : 0][k], sc[t]);
+            }
         }
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
+        for (int t = 0; t < 2; ++t) {
             const int j = k0 + t * 16 + lr;
             const bool seen = j < pos && (pos - j < a.window || j < a.keep);
 #pragma unroll
             for (int r = 0; r < 4; ++r) sc[t][r] = seen ? kv_score<T>(sc[t][r], cap, bias[t][r]) : -INFINITY;
         }
         weigh(sc);
+        Frag<T> pf[NP];
 #pragma unroll
-        for (int k = 0; k < 2; ++k) {
-            Frag<T> pf[NP];
+        for (int n = 0; n < NP; ++n) pf[n].load(P + (n * 16 + lr) * PS + lq * 8);
 #pragma unroll
-            for (int n = 0; n < NP; ++n) pf[n].load(P + (n * 16 + lr) * PS + k * 32 + lq * 8);
+        for (int j = 0; j < NV; ++j) {
+            if constexpr (!AHEAD) vf[j].load(V + (j * 16 + lr) * BAMD_PAGE + lq * 8);
 #pragma unroll
-            for (int j = 0; j < NV; ++j) {
-                Frag<T> vf; vf.load(V + (j * 16 + lr) * BAMD_PAGE + k * 32 + lq * 8);
-#pragma unroll
-                for (int n = 0; n < NP; ++n) o[j] = mma(pf[n], vf, o[j]);
-            }
+            for (int n = 0; n < NP; ++n) o[j] = mma(pf[n], vf[j], o[j]);
         }
         wave_lds_fence();
+        if (i + 1 < t1) request(i + 1);
     }
     if (own) {
-        Frag<T> kf[ND];
-        kv_head<T, ND>(a, in + a.k_off + g * D, lq, kf);           // the same in every column
-        bamd_v4 sc[4];
+        Frag<T> kn[ND];
+        kv_head_norm<T, ND>(a, kr, kn);
+        bamd_v4 sc[2];
         sc[0] = bamd_v4{ 0, 0, 0, 0 };
 #pragma unroll
-        for (int k = 0; k < ND; ++k) sc[0] = mma(q[k], kf[k], sc[0]);
+        for (int k = 0; k < ND; ++k) sc[0] = mma(q[k], kn[k], sc[0]);
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             sc[0][r] = lr == 0 ? kv_score<T>(sc[0][r], cap, kv_bias(a, h0 + min(lq * 4 + r, nh - 1), 0)) : -INFINITY;
-            sc[1][r] = sc[2][r] = sc[3][r] = -INFINITY;
+            sc[1][r] = -INFINITY;
         }
         weigh(sc);
         Frag<T> pf[NP];
 #pragma unroll
         for (int n = 0; n < NP; ++n) pf[n].load(P + (n * 16 + lr) * PS + lq * 8);
-        const float * v = in + a.v_off + g * D;
 #pragma unroll
         for (int j = 0; j < NV; ++j) {
-            Frag<T> vf; vf.zero();
-            if (lq == 0) vf.set(0, v[j * 16 + lr]);
+            Frag<T> vn; vn.zero();
+            if (lq == 0) vn.set(0, vr[j]);
 #pragma unroll
-            for (int n = 0; n < NP; ++n) o[j] = mma(pf[n], vf, o[j]);
+            for (int n = 0; n < NP; ++n) o[j] = mma(pf[n], vn, o[j]);
         }
         if (hg == 0) {                                             // into the cache; a page's first position also clears the places behind it
             const int off = pos % BAMD_PAGE;
             const size_t at = ((size_t) pages[pos / BAMD_PAGE] * a.kv_heads + g) * BAMD_PAGE * D;
             if (lr == 0)
 #pragma unroll
-                for (int k = 0; k < ND; ++k) kf[k].store((T *) a.kc + at + (size_t) off * D + k * 32 + lq * 8);
-            T * V = (T *) a.vc + at;
-            for (int d = lane; d < D; d += 64) {
-                if (off == 0) for (int c = 0; c < BAMD_PAGE * (int) sizeof(T) / 16; ++c) *(bamd_u4 *) ((unsigned char *) (V + (size_t) d * BAMD_PAGE) + c * 16) = bamd_u4{ 0, 0, 0, 0 };
-                V[(size_t) d * BAMD_PAGE + off] = to_act<T>(v[d]);
-            }
+                for (int k = 0; k < ND; ++k) kn[k].store((T *) a.kc + at + (size_t) off * D + k * 32 + lq * 8);
+            T * vd = (T *) a.vc + at;
+            if (off == 0) for (int c = lane; c < D * BAMD_PAGE * (int) sizeof(T) / 16; c += 64) if (c % (BAMD_PAGE * (int) sizeof(T) / 16)) ((bamd_u4 *) vd)[c] = bamd_u4{ 0, 0, 0, 0 };
+            if (lq == 0)
+#pragma unroll
+                for (int j = 0; j < NV; ++j) {
+                    T * row = vd + (size_t) (j * 16 + lr) * BAMD_PAGE;
+                    if (off == 0) { Frag<T> f; f.zero(); f.set(0, vr[j]); f.store(row); }       // (the first eight places)
+                    else row[off] = to_act<T>(vr[j]);
+                }
         }
     }
     // the four waves' sums

@@ -180,6 +180,9 @@ struct Timer {                                     // per-launch HIP events (pro
 };
 #define STACK_ROWS 2048                            /* token rows of one pass */
 #define SEG_MIN 64                                 /* tokens of the shortest scan segment */
+#ifndef PAIR_ROWS
+#define PAIR_ROWS 4                                /* decoding rows up to which two branches share their launches */
+#endif
 #define SEG_BLOCKS 768                             /* blocks a scan wants */
 struct Ctx {
     bamd_context * c = nullptr; Stack * st = nullptr;
@@ -328,7 +331,7 @@ std::vector<float> expand_bias(const std::vector<float> & rel, int rows, int hea
 }
 int kv_splits(const bamd_kv_args & a, int rows, int max_pages) {
     const int groups = std::max(1, rows * bamd_kv_groups(a)), span = bamd_kv_span(a, max_pages);
-    return std::max(1, std::min({ (span + 1 + 3) / 4, std::max(1, 1024 / groups), 64 }));        // four waves per share, the row's own key is one more page
+    return std::max(1, std::min({ (2 * span + 1 + 3) / 4, std::max(1, 1024 / groups), 64 }));    // four waves per share, half a page each; the row's own key is one more
 }
 struct KvAttention : Branch {
     bamd_kv_args a; int vdim = 0;
@@ -375,6 +378,7 @@ struct KvAttention : Branch {
     }
     int state(Ctx & c, MixState & st) override;
     int run(Pass & p, MixState & st, int ld, int ldo) override;
+    bamd_kv_args args(Pass & p, MixState & st, int ld, int ldo) const;
 };
 struct GatedLinear : Branch {
     bamd_gla_args a; int N = 0;
@@ -417,6 +421,7 @@ struct GatedLinear : Branch {
     int scan_blocks() const override { return bamd_gla_blocks(a.heads, a.Pp); }
     int state(Ctx & c, MixState & st) override;
     int run(Pass & p, MixState & st, int ld, int ldo) override;
+    bamd_gla_args args(Pass & p, MixState & st, int ld, int ldo) const;
 };
 // several branches over one input, their outputs summed with a scale each
 struct Parallel : Mixer {
@@ -669,11 +674,15 @@ int LatentAttention::run(Pass & p, MixState & st, Operand & o) {
     p.end();
     return rc ? fail("latent attention: unsupported shape") : 0;
 }
+bamd_kv_args KvAttention::args(Pass & p, MixState & st, int ld, int ldo) const {
+    bamd_kv_args k = a;
+    k.in = p.c.y; k.ld = ld; k.kc = st.cache; k.vc = st.cache2; k.out = p.c.h; k.ldo = ldo;
+    return k;
+}
 int KvAttention::run(Pass & p, MixState & st, int ld, int ldo) {
     Ctx & c = p.c;
     const int act = p.st.act;
-    bamd_kv_args k = a;
-    k.in = c.y; k.ld = ld; k.kc = st.cache; k.vc = st.cache2; k.out = c.h; k.ldo = ldo;
+    const bamd_kv_args k = args(p, st, ld, ldo);
     int rc = 0;
     if (p.decode) rc = bamd_launch_kv_decode(act, p.b, k, c.part_o, c.part_ml, kv_splits(k, p.b.rows, c.max_pages), p.s);
     else {
@@ -682,10 +691,14 @@ int KvAttention::run(Pass & p, MixState & st, int ld, int ldo) {
     }
     return rc ? fail("attention over keys and values: unsupported shape") : 0;
 }
+bamd_gla_args GatedLinear::args(Pass & p, MixState & st, int ld, int ldo) const {
+    bamd_gla_args g = a;
+    g.in = p.c.y; g.ld = ld; g.state = st.b; g.y = p.c.y3; g.ldy = a.heads * a.Pp; g.out = p.c.h; g.ldo = ldo;
+    return g;
+}
 int GatedLinear::run(Pass & p, MixState & st, int ld, int ldo) {
     Ctx & c = p.c;
-    bamd_gla_args g = a;
-    g.in = c.y; g.ld = ld; g.state = st.b; g.y = c.y3; g.ldy = a.heads * a.Pp; g.out = c.h; g.ldo = ldo;
+    bamd_gla_args g = args(p, st, ld, ldo);
     if (p.max_n > 1) {
         const size_t ch = (size_t) a.heads * a.Np;
         if (grow(c, (void **) &c.alpha, &c.alpha_n, (size_t) p.b.rows * ch * 4, p.s)) return 1;
@@ -699,7 +712,11 @@ int GatedLinear::run(Pass & p, MixState & st, int ld, int ldo) {
 int Parallel::run(Pass & p, MixState & st, Operand & o) {
     o.x = p.c.h; o.ldx = out.K;
     p.begin(1, p.tm ? step_bytes(p.c.seqs[0].len + 1) : 0);
-    for (size_t i = 0; i < br.size(); ++i) if (br[i]->run(p, st.sub[i], ld_of(in), out.K)) return 1;
+    auto * kv = dynamic_cast<KvAttention *>(br[0].get()); auto * gl = dynamic_cast<GatedLinear *>(br[1].get());
+    if (p.decode && p.b.rows <= PAIR_ROWS && kv && gl) {           // few rows: the branches' blocks share their launches
+        const bamd_kv_args k = kv->args(p, st.sub[0], ld_of(in), out.K);
+        if (bamd_launch_kv_gla_decode(p.st.act, p.b, k, gl->args(p, st.sub[1], ld_of(in), out.K), p.c.part_o, p.c.part_ml, kv_splits(k, p.b.rows, p.c.max_pages), p.s)) return fail("attention beside gated linear attention: unsupported shape");
+    } else for (size_t i = 0; i < br.size(); ++i) if (br[i]->run(p, st.sub[i], ld_of(in), out.K)) return 1;
     p.end();
     return 0;
 }
