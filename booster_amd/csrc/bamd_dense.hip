@@ -176,7 +176,7 @@ __global__ void __launch_bounds__(64 * NW) dense_mv_kernel(bamd_dense w, bamd_ba
         if constexpr (PRE == BAMD_PRE_RESIDUAL) residual_row<T, true>(b, p.res, 0, h, blockIdx.x == 0, red);
         if constexpr (PRE == BAMD_PRE_POLY) poly_row<T>(p.poly, 0, h, red);
         if constexpr (PRE == BAMD_PRE_GROUP) group_norm_row<T>(p.grp, 0, h, red);
-        if constexpr (PRE == BAMD_PRE_GLU) glu_row<T>(p.glu, 0, h);
+        if constexpr (PRE == BAMD_PRE_GLU) glu_row<T>(p.glu, 0, h, 0, p.glu.ldh);
         if constexpr (PRE == BAMD_PRE_LAYER) layer_row<T>(p.res, p.want ? p.want[0] : 0, p.want ? p.gf : p.res.gi, h, !p.want && blockIdx.x == 0, red);
         if constexpr (PRE == BAMD_PRE_FINAL) final_row<T>(p.res, p.want[0], p.gf, h, red);
         __syncthreads();

@@ -207,10 +207,11 @@ __device__ __forceinline__ float clamped_glu(float gate, float up, float limit) 
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
 }
+// columns [from, to) of a row
 template <typename T>
-__device__ __forceinline__ void glu_row(const bamd_glu_args & a, int row, T * h) {
+__device__ __forceinline__ void glu_row(const bamd_glu_args & a, int row, T * h, int from, int to) {
     const float * z = a.z + (size_t) row * a.ldz;
-    for (int i = threadIdx.x * 4; i < a.ldh; i += blockDim.x * 4) {
+    for (int i = from + threadIdx.x * 4; i < to; i += blockDim.x * 4) {
         const bamd_v4 g = *(const bamd_v4 *) (z + (i >> 4) * 32 + (i & 15)), u = *(const bamd_v4 *) (z + (i >> 4) * 32 + 16 + (i & 15));
         store4<T>(h + i, bamd_v4{ clamped_glu(g[0], u[0], a.limit), clamped_glu(g[1], u[1], a.limit), clamped_glu(g[2], u[2], a.limit), clamped_glu(g[3], u[3], a.limit) });
     }

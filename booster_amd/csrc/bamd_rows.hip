@@ -28,7 +28,8 @@ template <typename T> __global__ void __launch_bounds__(1024) layer_rows_kernel(
     const int row = want ? want[blockIdx.x] : blockIdx.x;
     layer_row<T>(a, row, gi, a.h ? (T *) a.h + (size_t) blockIdx.x * a.ldh : nullptr, !want, red);
 }
-template <typename T> __global__ void __launch_bounds__(256) glu_rows_kernel(bamd_glu_args a) { glu_row<T>(a, blockIdx.x, (T *) a.h + (size_t) blockIdx.x * a.ldh); }
+// block (1024 columns, row)
+template <typename T> __global__ void __launch_bounds__(256) glu_rows_kernel(bamd_glu_args a) { glu_row<T>(a, blockIdx.y, (T *) a.h + (size_t) blockIdx.y * a.ldh, blockIdx.x * 1024, min(a.ldh, (int) blockIdx.x * 1024 + 1024)); }
 template <typename T> __global__ void __launch_bounds__(1024) poly_rows_kernel(bamd_poly_args a) {
     __shared__ float red[64];
     poly_row<T>(a, blockIdx.x, (T *) a.h + (size_t) blockIdx.x * a.ldh, red);
@@ -92,8 +93,8 @@ void bamd_launch_poly_rows(int act, int rows, const bamd_poly_args & a, hipStrea
     else hipLaunchKernelGGL(poly_rows_kernel<bamd_bf>, dim3(rows), row_block(a.F), 0, s, a);
 }
 void bamd_launch_glu_rows(int act, int rows, const bamd_glu_args & a, hipStream_t s) {
-    if (act == BAMD_ACT_F32) hipLaunchKernelGGL(glu_rows_kernel<float>, dim3(rows), dim3(256), 0, s, a);
-    else hipLaunchKernelGGL(glu_rows_kernel<bamd_bf>, dim3(rows), dim3(256), 0, s, a);
+    if (act == BAMD_ACT_F32) hipLaunchKernelGGL(glu_rows_kernel<float>, dim3((a.ldh + 1023) / 1024, rows), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(glu_rows_kernel<bamd_bf>, dim3((a.ldh + 1023) / 1024, rows), dim3(256), 0, s, a);
 }
 void bamd_launch_group_norm_rows(int act, int rows, const bamd_group_norm_args & a, hipStream_t s) {
     if (act == BAMD_ACT_F32) hipLaunchKernelGGL(group_norm_rows_kernel<float>, dim3(rows), row_block(a.n), 0, s, a);
