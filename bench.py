@@ -582,8 +582,8 @@ def stack_configs(E, F, H, hd, R, mheads, P, state, gheads, gdim, gvdim, window,
     mlp = {"kind": "dense", "ff": F}
     at = {"type": "latent_attention", "mixer": dict(heads=H, dim=hd, vdim=hd, kv_rank=R, scale=hd ** -0.5), "mlp": mlp}
     mb = {"type": "mamba2", "mixer": dict(heads=mheads, vdim=P, state=state, groups=1, norm_groups=1, conv=4), "mlp": mlp}
-    left = dict(heads=H, kv_heads=H // 4, dim=hd, vdim=hd, scale=hd ** -0.5, softcap=20.0, bias_max=512, mask=dict(size=window, keep_first=4))
-    side = {"type": "parallel", "mixer": dict(left=left, left_scale=0.6, right=dict(heads=gheads, dim=gdim, vdim=gvdim, tau=16.0), right_scale=1.1), "mlp": dict(mlp, limit=7.0)}
+    left = dict(heads=H, kv_heads=H // 4, dim=hd, vdim=hd, scale=hd ** -0.5, softcap=30.0, bias_max=512, mask=dict(size=window, keep_first=4))
+    side = {"type": "parallel", "mixer": dict(left=left, left_scale=0.5, right=dict(heads=gheads, dim=gdim, vdim=gvdim, tau=16.0), right_scale=0.8), "mlp": dict(mlp, limit=7.0)}
     return {"stack": {"architecture": "Tupitar", "vocab": V, "width": E, "max_positions": max_positions, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6}, "layers": [at, mb] * (L // 2)},
             "mafurax": {"architecture": "Mafurax", "vocab": V, "width": E, "logit_scale": E ** -0.5, "norm": {"eps": 1e-6}, "layers": [side] * L}}
 

@@ -204,11 +204,11 @@ __global__ void __launch_bounds__(256) kv_prompt_kernel(bamd_batch_dev b, bamd_k
         }
 }
 
-// block (share, kv head and head group, row)
+// block (kv head and head group, share, row): where only some shares hold keys, their blocks still spread over all XCDs
 template <typename T, int ND>
-__global__ void __launch_bounds__(256) kv_decode_kernel(bamd_batch_dev b, bamd_kv_args a, float * part_o, float * part_ml, int splits) {
+__global__ void __launch_bounds__(256, ND <= 4 ? 2 : 1) kv_decode_kernel(bamd_batch_dev b, bamd_kv_args a, float * part_o, float * part_ml, int splits) {
     extern __shared__ __align__(16) unsigned char lds[];
-    kv_decode_block<T, ND>(b, a, blockIdx.x, splits, blockIdx.y, blockIdx.z, part_o, part_ml, lds);
+    kv_decode_block<T, ND>(b, a, blockIdx.y, splits, blockIdx.x, blockIdx.z, part_o, part_ml, lds);
 }
 template <typename T> __global__ void __launch_bounds__(256) kv_combine_kernel(bamd_kv_args a, const float * part_o, const float * part_ml, int splits) {
     kv_combine_block<T>(a, blockIdx.x, blockIdx.y, part_o, part_ml, splits);
@@ -255,7 +255,7 @@ int bamd_kv_span(const bamd_kv_args & a, int pages) {
 template <typename T, int ND>
 static int decode_go(const bamd_batch_dev & b, const bamd_kv_args & a, float * po, float * pm, int splits, hipStream_t s) {
     constexpr size_t lds = KvDecodeLds<T, ND>::bytes;
-    hipLaunchKernelGGL((kv_decode_kernel<T, ND>), dim3(splits, bamd_kv_groups(a), b.rows), dim3(256), lds, s, b, a, po, pm, splits);
+    hipLaunchKernelGGL((kv_decode_kernel<T, ND>), dim3(bamd_kv_groups(a), splits, b.rows), dim3(256), lds, s, b, a, po, pm, splits);
     hipLaunchKernelGGL(kv_combine_kernel<T>, dim3(a.heads, b.rows), dim3(a.D < 64 ? 64 : a.D), 0, s, a, po, pm, splits);
     return 0;
 }

@@ -73,6 +73,12 @@ __device__ __forceinline__ void kv_decode_block(const bamd_batch_dev & b, const 
     const KvPages pg(a, pos - a.window + 1, (pos + BAMD_PAGE - 1) / BAMD_PAGE);
     const int per = (2 * pg.count + nw - 1) / nw, t0 = wi * per, t1 = min(2 * pg.count, t0 + per);
     const bool own = wi == nw - 1;
+    const size_t base = ((size_t) row * a.kv_heads * hgs + y) * splits + sp;
+    if (sp * 4 * per >= 2 * pg.count && sp != splits - 1) {        // a share without keys
+        for (int i = tid; i < nh * D; i += 256) part_o[base * 16 * D + i] = 0.f;
+        if (tid < nh) { part_ml[(base * 16 + tid) * 2] = -INFINITY; part_ml[(base * 16 + tid) * 2 + 1] = 0.f; }
+        return;
+    }
     const int32_t * pages = b.pages + (size_t) e.seq * b.max_pages;
     const float * in = a.in + (size_t) row * a.ld;
     const KvCap cap = kv_cap(a);
@@ -221,7 +227,6 @@ __device__ __forceinline__ void kv_decode_block(const bamd_batch_dev & b, const 
         for (int j = 0; j < NV; ++j) so[((size_t) wave * 16 + hd) * D + j * 16 + lr] = o[j][r];
     }
     __syncthreads();
-    const size_t base = ((size_t) row * a.kv_heads * hgs + y) * splits + sp;
     for (int i = tid; i < nh * D; i += 256) {
         const int hd = i / D, d = i % D;
         float mx = -INFINITY, s = 0.f, t = 0.f;

@@ -10,7 +10,7 @@ template <typename T, int ND, int NPL>
 __global__ void __launch_bounds__(256, ND <= 4 ? 2 : 1) kv_gla_step_kernel(bamd_batch_dev b, bamd_kv_args kv, bamd_gla_args gla, float * part_o, float * part_ml, int splits, int attn) {
     extern __shared__ __align__(16) unsigned char lds[];
     const int x = blockIdx.x, row = blockIdx.y;
-    if (x < attn) { kv_decode_block<T, ND>(b, kv, x % splits, splits, x / splits, row, part_o, part_ml, lds); return; }
+    if (x < attn) { kv_decode_block<T, ND>(b, kv, x / (attn / splits), splits, x % (attn / splits), row, part_o, part_ml, lds); return; }
     const int cols = (gla.Pp + PAIR_PT - 1) / PAIR_PT, i = x - attn, h = i / cols;
     const bamd_entry e = b.ent[row];
     float * st = gla.state + ((size_t) e.seq * gla.heads + h) * gla.Np * gla.Pp;

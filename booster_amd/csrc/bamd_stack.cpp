@@ -1,5 +1,5 @@
 // bamd_stack.cpp — host runtime of configured layer stacks (bamd_stack.h): configuration, weights (safetensors -> packed matrices on the device), per-sequence
-// state (latent pages, recurrent and convolution states, previous inputs), the scheduler that cuts a batch into passes, and the passes themselves.
+// state (pages of latents or of keys and values, recurrent and convolution states, previous inputs), the scheduler that cuts a batch into passes, and the passes themselves.
 //
 // A context holds n_seq sequences over one pool of 64-position pages.  State that a pass both reads and replaces (previous inputs, convolution inputs) is double
 // buffered per sequence; the recurrent state is owned by one block and updated in place.  A pass runs either decoding rows (one token per sequence; replayed as a
@@ -178,11 +178,10 @@ struct Timer {                                     // per-launch HIP events (pro
     std::vector<hipEvent_t> ev; std::vector<int> kind; std::vector<double> bytes;
     ~Timer() { for (auto e : ev) hipEventDestroy(e); }
 };
+#define STACK_CTX 8192                             /* positions of a context that asks for none, where the model sets no bound */
 #define STACK_ROWS 2048                            /* token rows of one pass */
 #define SEG_MIN 64                                 /* tokens of the shortest scan segment */
-#ifndef PAIR_ROWS
 #define PAIR_ROWS 4                                /* decoding rows up to which two branches share their launches */
-#endif
 #define SEG_BLOCKS 768                             /* blocks a scan wants */
 struct Ctx {
     bamd_context * c = nullptr; Stack * st = nullptr;
@@ -482,7 +481,7 @@ int Stack::load(bamd_model * model, const bamd_load_args & a, const bamd_stack_d
     int lf = a.layer_first, ll = a.layer_last;
     if (ll < 0 || ll > L) ll = L;
     if (lf < 0 || lf > ll) return fail("bad layer range");
-    m->E = E; m->V = V; m->L = L; m->eps = eps; m->n_ctx_train = max_pos; m->layer_first = lf; m->layer_last = ll; m->with_embd = a.with_embd != 0; m->with_output = a.with_output != 0;
+    m->E = E; m->V = V; m->L = L; m->eps = eps; m->n_ctx_train = d.learned_positions ? max_pos : STACK_CTX; m->layer_first = lf; m->layer_last = ll; m->with_embd = a.with_embd != 0; m->with_output = a.with_output != 0;
     if (a.dtype != BAMD_DTYPE_DEFAULT && a.dtype != BAMD_DTYPE_BF16 && a.dtype != BAMD_DTYPE_F32) return fail("unknown dtype");
     act = a.dtype == BAMD_DTYPE_F32 ? BAMD_ACT_F32 : BAMD_ACT_BF16;
     { std::ifstream v(dir + "/tokenizer.gguf"); if (v) vocab = dir + "/tokenizer.gguf"; }

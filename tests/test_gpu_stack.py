@@ -479,28 +479,32 @@ def test_replays_with_other_work_between(bamd, cases, name):
     c.close(); m.close()
 
 
-def test_bridge_serves_a_model_folder(bamd, tmp_path):
+@pytest.mark.parametrize("design", ["Tupitar", "Mafurax"])
+def test_bridge_serves_a_model_folder(bamd, design, tmp_path):
     """initContext / doInference on a folder with tokenizer.gguf: prompt, Janus sampling on the device's logits, text out; without a tokenizer the request is refused"""
     from booster_amd import gguf
     from test_gpu_bridge import bind, ctx_args
     L = bind(bamd)
     vocab = gguf.synthetic_spm_vocab()
     cfg = config(60, len(vocab["tokens"]), [mamba(2, 12, 16, 1, 2, 4, ff=50), latent(3, 16, 20, 24, 0.3, ff=64)], max_positions=192)
+    if design == "Mafurax":
+        cfg = mafurax(60, len(vocab["tokens"]), [parallel(attend(4, 2, 16, 20, 0.4, 7.0, 30, 9, 2), 0.9, (2, 12, 16, 4.0), 0.8, ff=50, limit=0.9)])
+    jobs = [(design + n).encode() for n in ("-none", "-a", "-b")]
     d = str(tmp_path / "m")
     so.write_model(d, cfg, so.random_model(cfg, 8))
     ctx = L.initContext(*ctx_args(6, d, (100, 0, 0, 0), 128, 24))
-    assert ctx and L.doInference(6, ctx, b"stack-none", b"s", b"the cat sat") == 1
+    assert ctx and L.doInference(6, ctx, jobs[0], b"s", b"the cat sat") == 1
     gguf.write_synthetic_llama(d + "/tokenizer.gguf", E=256, H=2, Hkv=1, L=1, F=256, V=len(vocab["tokens"]), seed=2, vocab=vocab)
     ctx = L.initContext(*ctx_args(6, d, (100, 0, 0, 0), 128, 24))
     assert ctx
-    for job in (b"stack-a", b"stack-b"):                  # the second request starts over in the same context
+    for job in jobs[1:]:                  # the second request starts over in the same context
         n = L.doInference(6, ctx, job, b"s", b"the cat sat on the hat")
         prompt = L.getPromptTokenCount(job)
         assert prompt > 4 and prompt <= n <= prompt + 23
         text = L.status(job)
         assert b"the cat sat on the hat" in text
     # hi = lo = 1: only the top candidate survives, the draw is the arg-max of the penalised logits and both requests agree
-    assert L.status(b"stack-a") == L.status(b"stack-b")
+    assert L.status(jobs[1]) == L.status(jobs[2])
 
 
 @pytest.mark.parametrize("name", ["odd", "side"])
